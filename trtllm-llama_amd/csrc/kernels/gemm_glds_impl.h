@@ -3,6 +3,7 @@
 // one source.  Everything has internal linkage.
 #pragma once
 #include "dev_utils.h"
+#include "gemm_seam.h"
 #include "kernels.h"
 #include "launch_util.h"
 
@@ -80,7 +81,10 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
             p.M = p.group_off[blockIdx.y + 1] - (int) o;
             if (p.M <= 0)
                 return;
-            p.a = reinterpret_cast<const char*>(p.a) + o * p.lda * 2;
+            if (p.a_rows)
+                p.a_rows += o;
+            else
+                p.a = reinterpret_cast<const char*>(p.a) + o * p.lda * 2;
             p.c = reinterpret_cast<char*>(p.c) + o * p.ldc * (p.out_dtype == DT_FLOAT ? 4 : 2);
         }
     }
@@ -152,7 +156,12 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
         const int col = BKB == 128 ? (lane & 7) ^ ((row >> 1) & 7) : (lane & 3) ^ ((row >> 2) & 3);
         if (row < BM)
         {
-            const int gr = m0 + row < M ? m0 + row : M - 1;
+            int gr = m0 + row < M ? m0 + row : M - 1;
+            if constexpr (WT == W_BF16)
+            {
+                if (p.a_rows)
+                    gr = p.a_rows[gr];
+            }
             if constexpr (LW > 0)
                 soff[i] = (uint32_t) ((int64_t) gr * p.lda * ES + col * 16);
             else
@@ -210,8 +219,20 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                 acc[i][j][r] = 0;
 
     const int fr = lane & 31, fk = lane >> 5;
-    const bool vec_out = p.out_dtype == (WT == W_BF16 ? DT_BFLOAT16 : DT_HALF) && !p.resid && !p.bias && !p.act && !(p.ldc & 7) && !(N & 7) && !(reinterpret_cast<uintptr_t>(p.c) & 15)
+    bool vec_out = p.out_dtype == (WT == W_BF16 ? DT_BFLOAT16 : DT_HALF) && !p.resid && !p.bias && (!p.act || (WT == W_BF16 && p.act == GEMM_ACT_RELU2)) && !(p.ldc & 7) && !(N & 7) && !(reinterpret_cast<uintptr_t>(p.c) & 15)
         && !(reinterpret_cast<uintptr_t>(p.residual) & 15);
+    if constexpr (WT == W_BF16)
+    {
+        // columns that leave through an output section of their own go in the same 16-byte pieces where its rows allow it; a tile that
+        // reaches a section of fp32 columns stores element by element
+        auto sec_ok = [&](const GemmSection& sc) {
+            return n0 + BN <= sc.col0 || (!sc.f32 && !(sc.col0 & 7) && !(reinterpret_cast<uintptr_t>(sc.c) & 15) && !(sc.ldc & 7));
+        };
+        if (p.seam.n_sec > 0)
+            vec_out = vec_out && sec_ok(p.seam.sec[0]);
+        if (p.seam.n_sec > 1)
+            vec_out = vec_out && sec_ok(p.seam.sec[1]);
+    }
     if constexpr (LW > 0)
     {
         // the loaders' whole life: request, wait, barrier, request ... - a loop of its own, so that none of the compute waves'
@@ -392,6 +413,10 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
         constexpr int PITCH = NT * 64 + 16;
         __syncthreads(); // every wave has finished reading the operand buffers
         char* scr = lds + wid * (32 * PITCH);
+        bool relu2_col[NT];
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+            relu2_col[j] = WT == W_BF16 && seam_out<false>(p.seam, p.act, p.c, p.ldc, false, wave_n0 + j * 32 + (lane & 31)).act == GEMM_ACT_RELU2;
 #pragma unroll
         for (int i = 0; i < MT; ++i)
         {
@@ -413,6 +438,11 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                     }
                     else
                         v = acc[i][j][r] * sc[j];
+                    if constexpr (WT == W_BF16)
+                    {
+                        if (relu2_col[j])
+                            v = seam_relu2(bf2f(f2bf(v)));
+                    }
                     *reinterpret_cast<uint16_t*>(scr + rr * PITCH + (j * 32 + (lane & 31)) * 2) = WT == W_BF16 ? f2bf(v) : f2h(v);
                 }
             // 32 rows x (NT * 4) 16-byte pieces
@@ -426,6 +456,12 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                 if (grow < M && gcol < N)
                 {
                     const int64_t o = (int64_t) grow * p.ldc + gcol;
+                    uint16_t* dst = reinterpret_cast<uint16_t*>(p.c) + o;
+                    if constexpr (WT == W_BF16)
+                    {
+                        const SeamOut so = seam_out<false>(p.seam, p.act, p.c, p.ldc, false, gcol);
+                        dst = reinterpret_cast<uint16_t*>(so.c) + (int64_t) grow * so.ldc + gcol;
+                    }
                     if (p.residual)
                     {
                         const uint4 rv = *reinterpret_cast<const uint4*>(reinterpret_cast<const uint16_t*>(p.residual) + o);
@@ -439,7 +475,7 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                     }
                     else if (p.silu_gate)
                         v = epi_silu_gate8(v, *reinterpret_cast<const uint4*>(reinterpret_cast<const uint16_t*>(p.silu_gate) + o));
-                    *reinterpret_cast<uint4*>(reinterpret_cast<uint16_t*>(p.c) + o) = v;
+                    *reinterpret_cast<uint4*>(dst) = v;
                 }
             }
         }
@@ -453,6 +489,9 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
             const int col = wave_n0 + j * 32 + (lane & 31);
             if (col >= N || i < i_lo || i >= i_hi)
                 continue;
+            SeamOut so{};
+            if constexpr (WT == W_BF16)
+                so = seam_out<false>(p.seam, p.act, p.c, p.ldc, p.out_dtype != DT_BFLOAT16, col);
 #pragma unroll
             for (int r = 0; r < 16; ++r)
             {
@@ -491,17 +530,7 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                     }
                     else
                     {
-                        float u = p.bias ? v + p.bias[col] : v;
-                        if (p.act == 1)
-                        {
-                            u = p.out_dtype == DT_BFLOAT16 ? bf2f(f2bf(u)) : u;
-                            u = fmaxf(u, 0.f);
-                            u *= u;
-                        }
-                        if (p.out_dtype == DT_BFLOAT16)
-                            reinterpret_cast<uint16_t*>(p.c)[o] = f2bf(u);
-                        else
-                            reinterpret_cast<float*>(p.c)[o] = u;
+                        seam_store<false, (MT * NT <= 4)>(p.seam, so, row, col, p.bias ? v + p.bias[col] : v);
                     }
                 }
                 else

@@ -15,6 +15,7 @@
 // Fragment layouts (gfx950): A/B operand of a 32x32xK MFMA: lane l holds row (l & 31), k-bytes [16*(l>>5), +16) of the
 // K-slab's 32-byte half; C/D: col = l & 31, row = (r & 3) + 8 * (r >> 2) + 4 * (l >> 5).
 #include "dev_utils.h"
+#include "gemm_seam.h"
 #include "kernels.h"
 #include "weight_layout.h"
 
@@ -245,6 +246,9 @@ __global__ __launch_bounds__(256) void gemm_mfma_kernel(const GemmParams p)
                 sc = p.per_channel ? reinterpret_cast<const float*>(p.scale_col)[col] : reinterpret_cast<const float*>(p.scale_col)[0];
             else if constexpr (WT == W_INT8_WOQ || WT == W_INT4_WOQ)
                 sc = h2f(reinterpret_cast<const uint16_t*>(p.scale_col)[col]);
+            SeamOut so{};
+            if constexpr (WT == W_BF16)
+                so = seam_out<false>(p.seam, p.act, p.c, p.ldc, p.out_dtype != DT_BFLOAT16, col);
 #pragma unroll
             for (int r = 0; r < 16; ++r)
             {
@@ -282,17 +286,7 @@ __global__ __launch_bounds__(256) void gemm_mfma_kernel(const GemmParams p)
                     }
                     else
                     {
-                        float u = p.bias ? v + p.bias[col] : v;
-                        if (p.act == 1)
-                        {
-                            u = p.out_dtype == DT_BFLOAT16 ? bf2f(f2bf(u)) : u;
-                            u = fmaxf(u, 0.f);
-                            u *= u;
-                        }
-                        if (p.out_dtype == DT_BFLOAT16)
-                            reinterpret_cast<uint16_t*>(p.c)[o] = f2bf(u);
-                        else
-                            reinterpret_cast<float*>(p.c)[o] = u;
+                        seam_store<false>(p.seam, so, row, col, p.bias ? v + p.bias[col] : v);
                     }
                 }
                 else

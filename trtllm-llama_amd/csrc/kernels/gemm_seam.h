@@ -1,0 +1,93 @@
+// How a finished element of a stack-engine product leaves (stack_kernels.h, StackGemmParams): shared by the fp32 FMA tiles, the skinny
+// kernel and both MFMA tile kernels.
+#pragma once
+#include "dev_utils.h"
+#include "kernels.h"
+
+namespace tllm
+{
+namespace dev
+{
+using namespace kernels;
+
+template <bool F32>
+__device__ __forceinline__ float seam_ld(const void* p, int64_t i)
+{
+    if constexpr (F32)
+        return reinterpret_cast<const float*>(p)[i];
+    else
+        return bf2f(reinterpret_cast<const uint16_t*>(p)[i]);
+}
+
+__device__ __forceinline__ float seam_relu2(float v)
+{
+    v = fmaxf(v, 0.f);
+    return v * v;
+}
+
+// Where an element of column `col` goes and through which activation: the product's own c, or an output section (resolved once per
+// column; no array is indexed at run time, so the parameters stay in scalar registers).
+struct SeamOut
+{
+    void* c;     // element (row, col) at row * ldc + col
+    int64_t ldc;
+    int act;
+    bool f32;
+};
+template <bool EL_F32>
+__device__ __forceinline__ SeamOut seam_out(const GemmSeam& s, int act, void* c, int64_t ldc, bool c_f32, int col)
+{
+    SeamOut o{c, ldc, act, EL_F32 || c_f32};
+    int col0 = 0;
+    if (s.n_sec > 0 && col >= s.sec[0].col0)
+    {
+        o = SeamOut{s.sec[0].c, s.sec[0].ldc, s.sec[0].act, EL_F32 || s.sec[0].f32};
+        col0 = s.sec[0].col0;
+    }
+    if (s.n_sec > 1 && col >= s.sec[1].col0)
+    {
+        o = SeamOut{s.sec[1].c, s.sec[1].ldc, s.sec[1].act, EL_F32 || s.sec[1].f32};
+        col0 = s.sec[1].col0;
+    }
+    o.c = reinterpret_cast<char*>(o.c) - (int64_t) col0 * (o.f32 ? 4 : 2);
+    return o;
+}
+
+// v: the accumulator, bias already added.  ALL_ACTS: the activations beyond relu^2 are compiled in (the tile kernels with many accumulators
+// per lane leave them to the smaller shapes: their unrolled epilogue would not fit)
+template <bool EL_F32, bool ALL_ACTS = true>
+__device__ __forceinline__ void seam_store(const GemmSeam& s, const SeamOut& o, int row, int col, float v)
+{
+    if (o.act != GEMM_ACT_NONE)
+    {
+        if (o.act == GEMM_ACT_RELU2)
+            v = seam_relu2(o.f32 ? v : bf2f(f2bf(v))); // the projection's value in its element type, then its activation
+        else if (!ALL_ACTS)
+            ;
+        else if (o.act == GEMM_ACT_SCALE_CAP)
+        {
+            v *= s.act_scale;
+            if (s.act_cap > 0.f)
+            {
+                if constexpr (EL_F32)
+                    v = s.act_cap * tanhf(v / s.act_cap);
+                else
+                    v = s.act_cap * (1.f - 2.f / (1.f + __expf(2.f * v / s.act_cap))); // tanh y = 1 - 2 / (1 + e^2y)
+            }
+        }
+        else
+        {
+            const float z = o.f32 ? v : bf2f(f2bf(v));
+            const float u = 2.f * 0.7978845608028654f * (z + 0.044715f * z * z * z); // (1 + tanh(u / 2)) / 2 = 1 / (1 + e^-u)
+            v = z / (1.f + (EL_F32 ? expf(-u) : __expf(-u))) * seam_ld<EL_F32>(s.mul, (int64_t) s.mul_rows[row] * s.ld_mul + col);
+        }
+    }
+    const int64_t at = (int64_t) row * o.ldc + col;
+    if (o.f32)
+        reinterpret_cast<float*>(o.c)[at] = v;
+    else
+        reinterpret_cast<uint16_t*>(o.c)[at] = f2bf(v);
+}
+
+} // namespace dev
+} // namespace tllm

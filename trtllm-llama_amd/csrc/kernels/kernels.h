@@ -327,6 +327,30 @@ int launch_context_attention(const ContextAttnParams& p, hipStream_t stream);
 // ---------------------------------------------------------------------------------------------
 // MFMA GEMMs for M > 8 (prefill): C[m,n] = sum_k A[m,k] * B[n,k].
 // ---------------------------------------------------------------------------------------------
+// What a bfloat16 product of the stack engine may do with its result besides a plain store (gemm_seam.h applies it).
+constexpr int32_t GEMM_ACT_NONE = 0;
+constexpr int32_t GEMM_ACT_RELU2 = 1;     // max(v, 0)^2 of the value rounded to the output type
+constexpr int32_t GEMM_ACT_SCALE_CAP = 2; // v * act_scale, then act_cap * tanh(v / act_cap) where act_cap > 0
+constexpr int32_t GEMM_ACT_GELU_MUL = 3;  // gelu_tanh(v of the output type) * mul[mul_rows[m], n]
+struct GemmSection
+{
+    int32_t col0 = 0;  // first column of the section (the section before it ends here)
+    void* c = nullptr; // [M, ldc]; column n goes to c[m, n - col0]
+    int64_t ldc = 0;
+    int32_t act = GEMM_ACT_NONE; // NONE or RELU2
+    int32_t f32 = 0;             // c is fp32
+};
+struct GemmSeam
+{
+    float act_scale = 1.f, act_cap = 0.f;
+    const void* mul = nullptr; // table of the element type, rows of ld_mul elements
+    const int32_t* mul_rows = nullptr;
+    int64_t ld_mul = 0;
+    // columns from sec[i].col0 on leave through sec[i] (ascending; a layer's projections that read the same input but go different ways)
+    int32_t n_sec = 0;
+    GemmSection sec[2];
+};
+
 struct GemmParams
 {
     int32_t wtype = W_FP16; // same weight layouts as GemvParams
@@ -359,9 +383,11 @@ struct GemmParams
     const void* gate = nullptr;
     int64_t ldg = 0;
     const float* gate_bias = nullptr;
-    // W_BF16 only, without resid: + bias[n] (fp32 [N]) on the accumulator; act 1: max(v, 0)^2 of the value rounded to the output type
+    // W_BF16 only, without resid: + bias[n] (fp32 [N]) on the accumulator, then `act` (GEMM_ACT_*); `seam` holds its operands and the
+    // output sections of the columns behind the first ones
     const float* bias = nullptr;
     int32_t act = 0;
+    GemmSeam seam;
     // W_BF16 on the LDS-DMA tiles only: `batch` products of this shape in one launch, operands of product b at a + b * batch_a bytes,
     // w + b * batch_w, c + b * batch_c (no resid / residual)
     int32_t batch = 1;
@@ -369,6 +395,7 @@ struct GemmParams
     // ... grouped: device int32 [batch + 1]; product b takes rows [group_off[b], group_off[b + 1]) of a and c (batch_a = batch_c = 0), M
     // is the host's bound on a group's rows
     const int32_t* group_off = nullptr;
+    const int32_t* a_rows = nullptr; // grouped: row r of the products' common row range reads a's row a_rows[r]
     // microbench hook (tllm_gemm_set_clock_probe), set by the launchers only: 2 x uint64 per workgroup {shader cycles, 100 MHz ticks}
     void* clock_probe = nullptr;
     // split-K-2 forms of gemm_sqp.hip (r06), set by the launcher only: per tile two slabs of AH x BN accumulators + two flag words

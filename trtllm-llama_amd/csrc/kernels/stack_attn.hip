@@ -28,6 +28,7 @@ namespace
 constexpr int kSplitRows = 64, kMaxSplits = 16;
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4))); // staging registers: arrays of HIP's uint4 end up in scratch memory
 
 __device__ __forceinline__ bf16x8 as_bf16x8(const uint4& u)
 {
@@ -236,7 +237,7 @@ __global__ __launch_bounds__(NW * 64) void attn_tile_kernel(const StackAttnParam
     // ks == 1: blockIdx.x is the entry's 16-row tile.  ks > 1 (decoding steps: every entry one tile): blockIdx.x is the key split -
     // workgroup `split` of an (entry, head) takes the key blocks split * NW + w, + ks * NW, ... and leaves an unnormalised partial
     // (max, sum, O per map and row) in split_ws; attn_split_merge_kernel finishes the rows.
-    // head_rows (a step of single decoded tokens whose heads all share ONE key/value head and have no numbers of their own): the
+    // head_rows (a step of single decoded tokens whose heads all share ONE key/value head and have no numbers inside the score): the
     // tile's 16 rows are 16 HEADS of the entry's one token, blockIdx.z the group of heads - the keys are walked once per 16 heads
     const int e = blockIdx.y, hbase = head_rows ? blockIdx.z * 16 : 0, h = head_rows ? hbase : blockIdx.z;
     const int r0 = (ks > 1 || head_rows) ? 0 : blockIdx.x * 16;
@@ -405,7 +406,7 @@ __global__ __launch_bounds__(NW * 64) void attn_tile_kernel(const StackAttnParam
         }
         else
         {
-            const float fin = finish_factor(p, h, M, L);
+            const float fin = finish_factor(p, out_h < p.heads ? out_h : p.heads - 1, M, L);
 #pragma unroll
             for (int ww = 0; ww < NW; ++ww)
                 wgt[m][ww] *= fin;
@@ -541,7 +542,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const StackAttnParams
             acc[m][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 
-    uint4 kr[KPT], vr[VPT];
+    u32x4 kr[KPT], vr[VPT];
     // the page id of a block is fetched one block before its rows are requested: one memory latency per block, not two in a row
     const BlockWalk bw = block_walk(p, pos0 + tile * 64, nblk);
     // blocks below this index hold kept first keys, which every row sees whatever its own window (a wave whose rows start further
@@ -559,7 +560,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const StackAttnParams
             if (K16 % 256 == 0 || idx < K16)
             {
                 const int row = idx / (D / 8), piece = idx % (D / 8); // row = map * 32 + key
-                kr[i] = *reinterpret_cast<const uint4*>(
+                kr[i] = *reinterpret_cast<const u32x4*>(
                     kp + (((int64_t) blk * (p.kv_heads * MAPS) + g * MAPS + row / 32) * page + off + row % 32) * D + piece * 8);
             }
         }
@@ -568,7 +569,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const StackAttnParams
         {
             const int idx = tid + i * 256;
             if (V16 % 256 == 0 || idx < V16)
-                vr[i] = *reinterpret_cast<const uint4*>(vp + (((int64_t) blk * p.kv_heads + gv) * V + idx / 4) * page + off + (idx % 4) * 8);
+                vr[i] = *reinterpret_cast<const u32x4*>(vp + (((int64_t) blk * p.kv_heads + gv) * V + idx / 4) * page + off + (idx % 4) * 8);
         }
     };
     request(0);
@@ -580,14 +581,14 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const StackAttnParams
         {
             const int idx = tid + i * 256;
             if (K16 % 256 == 0 || idx < K16)
-                *reinterpret_cast<uint4*>(k_s + (idx / (D / 8)) * KP + (idx % (D / 8)) * 16) = kr[i];
+                *reinterpret_cast<u32x4*>(k_s + (idx / (D / 8)) * KP + (idx % (D / 8)) * 16) = kr[i];
         }
 #pragma unroll
         for (int i = 0; i < VPT; ++i)
         {
             const int idx = tid + i * 256;
             if (V16 % 256 == 0 || idx < V16)
-                *reinterpret_cast<uint4*>(v_s + (idx / 4) * VP + (idx % 4) * 16) = vr[i];
+                *reinterpret_cast<u32x4*>(v_s + (idx / 4) * VP + (idx % 4) * 16) = vr[i];
         }
         __syncthreads();
         if (vb + 1 < bw.n)
@@ -726,7 +727,7 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
     const int nblk = (pos0 + wg_last) / 32 + 1;
     const int wg_lo = first_visible(p, pos0 + tile * ROWS) / 32;
 
-    uint4 kr[KPT], vr[VPT];
+    u32x4 kr[KPT], vr[VPT];
     const BlockWalk bw = block_walk(p, pos0 + tile * ROWS, nblk);
     // blocks below this index hold kept first keys, which every row sees whatever its own window (a wave whose rows start further
     // down than the workgroup's first takes part in them too)
@@ -743,7 +744,7 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
             if (K16 % 256 == 0 || idx < K16)
             {
                 const int row = idx / (D / 8), piece = idx % (D / 8);
-                kr[i] = *reinterpret_cast<const uint4*>(kp + (((int64_t) blk * p.kv_heads + g) * page + off + row) * D + piece * 8);
+                kr[i] = *reinterpret_cast<const u32x4*>(kp + (((int64_t) blk * p.kv_heads + g) * page + off + row) * D + piece * 8);
             }
         }
 #pragma unroll
@@ -751,7 +752,7 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
         {
             const int idx = tid + i * 256;
             if (V16 % 256 == 0 || idx < V16)
-                vr[i] = *reinterpret_cast<const uint4*>(vp + (((int64_t) blk * p.kv_heads + gv) * V + idx / 4) * page + off + (idx % 4) * 8);
+                vr[i] = *reinterpret_cast<const u32x4*>(vp + (((int64_t) blk * p.kv_heads + gv) * V + idx / 4) * page + off + (idx % 4) * 8);
         }
     };
     request(0);
@@ -763,14 +764,14 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
         {
             const int idx = tid + i * 256;
             if (K16 % 256 == 0 || idx < K16)
-                *reinterpret_cast<uint4*>(k_s + (idx / (D / 8)) * KP + (idx % (D / 8)) * 16) = kr[i];
+                *reinterpret_cast<u32x4*>(k_s + (idx / (D / 8)) * KP + (idx % (D / 8)) * 16) = kr[i];
         }
 #pragma unroll
         for (int i = 0; i < VPT; ++i)
         {
             const int idx = tid + i * 256;
             if (V16 % 256 == 0 || idx < V16)
-                *reinterpret_cast<uint4*>(v_s + (idx / 4) * VP + (idx % 4) * 16) = vr[i];
+                *reinterpret_cast<u32x4*>(v_s + (idx / 4) * VP + (idx % 4) * 16) = vr[i];
         }
         __syncthreads();
         if (vb + 1 < bw.n)
@@ -956,8 +957,9 @@ int launch_tile(const StackAttnParams& p, hipStream_t stream)
             const int nblk = (span + 31) / 32;
             ks = std::min(kMaxSplits, (nblk + 2 * NW - 1) / (2 * NW));
         }
-        // single decoded tokens whose heads share one key/value head and carry no per-head numbers: 16 heads are the tile's rows
-        const int head_rows = (p.max_count == 1 && p.kv_heads == 1 && !p.cross_values && MAPS == 1 && p.heads >= 8 && !p.temp && !p.slope && !p.log_r1 && !p.sink
+        // single decoded tokens whose heads share one key/value head and carry no per-head score numbers: 16 heads are the tile's rows
+        // (a sink or an output gate is looked up per row)
+        const int head_rows = (p.max_count == 1 && p.kv_heads == 1 && !p.cross_values && MAPS == 1 && p.heads >= 8 && !p.temp && !p.slope && !p.log_r1
                                   && !p.wbias && !p.head_norm)
             ? 1
             : 0;
@@ -994,6 +996,14 @@ int launch_tile_latent(const StackAttnParams& p, hipStream_t stream)
         return launch_tile<1, 5, 8>(p, stream);
     if (p.dim == 320 && p.vdim == 256)
         return launch_tile<1, 10, 16>(p, stream);
+    // no rotated part: the key row is the latent alone (32, 64 and 128 are the ordinary shapes)
+    if (p.dim == p.vdim)
+        switch (p.dim)
+        {
+        case 96: return launch_tile<1, 3, 6>(p, stream);
+        case 192: return launch_tile<1, 6, 12>(p, stream);
+        case 256: return launch_tile<1, 8, 16>(p, stream);
+        }
     return 1;
 }
 
@@ -1021,7 +1031,8 @@ size_t stack_attn_workspace_floats(int32_t heads, int32_t maps, int32_t vdim)
 bool stack_attention_tiled(const StackAttnParams& p)
 {
     const bool std_shape = (p.dim == 32 || p.dim == 64 || p.dim == 128) && (p.vdim == 32 || p.vdim == 64 || p.vdim == 128);
-    const bool latent_shape = p.maps == 1 && p.kv_heads == 1 && ((p.dim == 160 && p.vdim == 128) || (p.dim == 320 && p.vdim == 256));
+    const bool latent_shape = p.maps == 1 && p.kv_heads == 1 && ((p.dim == 160 && p.vdim == 128) || (p.dim == 320 && p.vdim == 256)
+                                  || (p.dim == p.vdim && (p.dim == 96 || p.dim == 192 || p.dim == 256)));
     // what only the general kernels do: head-mixed weights, a gate per channel, kept first keys under a window
     if (p.talk || (p.out_gate && p.gate_wide))
         return false;

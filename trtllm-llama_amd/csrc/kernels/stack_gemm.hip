@@ -9,6 +9,7 @@
 //                     also the fallback for bfloat16 operands whose rows are not 16-byte aligned.
 #include "dev_utils.h"
 #include "gemm_glds_impl.h"
+#include "gemm_seam.h"
 #include "stack_kernels.h"
 #include <cstdlib>
 
@@ -47,19 +48,9 @@ __device__ __forceinline__ void seam(const StackGemmParams& p, int row, int col,
     }
     else
     {
-        const bool narrow = !(p.out_f32 || DT == DT_FLOAT);
         if (p.bias)
             v += p.bias[col];
-        if (p.act == ACT_RELU2)
-        {
-            v = narrow ? bf2f(f2bf(v)) : v; // the projection's value in its element type, then its activation
-            v = fmaxf(v, 0.f);
-            v *= v;
-        }
-        if (narrow)
-            reinterpret_cast<uint16_t*>(p.c)[(int64_t) row * p.ldc + col] = f2bf(v);
-        else
-            reinterpret_cast<float*>(p.c)[(int64_t) row * p.ldc + col] = v;
+        seam_store<DT == DT_FLOAT>(p.seam, seam_out<DT == DT_FLOAT>(p.seam, p.act, p.c, p.ldc, p.out_f32 != 0, col), row, col, v);
     }
 }
 
@@ -78,7 +69,10 @@ __device__ __forceinline__ StackGemmParams batch_slice(StackGemmParams p)
         // grouped form: this product's rows are a range of a and c that the device knows
         const int64_t o = p.group_off[b];
         p.M = p.group_off[b + 1] - (int) o;
-        p.a = reinterpret_cast<const char*>(p.a) + o * p.lda * ES;
+        if (p.a_rows)
+            p.a_rows += o;
+        else
+            p.a = reinterpret_cast<const char*>(p.a) + o * p.lda * ES;
         if (p.c)
             p.c = reinterpret_cast<char*>(p.c) + o * p.ldc * ((p.out_f32 || DT == DT_FLOAT) ? 4 : 2);
     }
@@ -91,12 +85,16 @@ template <int DT>
 __global__ __launch_bounds__(256) void fma_tile_kernel(const StackGemmParams p_in)
 {
     const StackGemmParams p = batch_slice<DT>(p_in);
+    __shared__ int64_t row_s[TM]; // where the tile's rows of a start
     __shared__ float As[TK][TM + 4];
     __shared__ float Ws[TK][TN + 4];
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
     const int m0 = blockIdx.y * TM, n0 = blockIdx.x * TN;
     if (m0 >= p.M)
         return; // (a group with fewer rows than the launch's bound)
+    if (tid < TM)
+        row_s[tid] = m0 + tid < p.M ? (int64_t) (p.a_rows ? p.a_rows[m0 + tid] : m0 + tid) * p.lda : 0;
+    __syncthreads();
     float acc[4][4];
 #pragma unroll
     for (int i = 0; i < 4; ++i)
@@ -109,7 +107,7 @@ __global__ __launch_bounds__(256) void fma_tile_kernel(const StackGemmParams p_i
         for (int i = 0; i < 4; ++i)
         {
             const int idx = tid + i * 256, r = idx / TK, k = idx % TK;
-            As[k][r] = (m0 + r < p.M && k0 + k < p.K) ? ld_el<DT>(p.a, (int64_t) (m0 + r) * p.lda + k0 + k) : 0.f;
+            As[k][r] = (m0 + r < p.M && k0 + k < p.K) ? ld_el<DT>(p.a, row_s[r] + k0 + k) : 0.f;
             Ws[k][r] = (n0 + r < p.N && k0 + k < p.K) ? ld_el<DT>(p.w, (int64_t) (n0 + r) * p.K + k0 + k) : 0.f;
         }
         __syncthreads();
@@ -160,6 +158,10 @@ __global__ __launch_bounds__(256) void skinny_kernel(const StackGemmParams p_in)
         for (int m = 0; m < MR; ++m)
             acc[r][m] = 0.f;
     const uint16_t* a = reinterpret_cast<const uint16_t*>(p.a);
+    int64_t arow[MR]; // where the rows of a start (p.M of them)
+#pragma unroll
+    for (int m = 0; m < MR; ++m)
+        arow[m] = m < p.M ? (int64_t) (p.a_rows ? p.a_rows[m] : m) * p.lda : 0;
     const uint16_t* w = reinterpret_cast<const uint16_t*>(p.w);
     for (int k = lane * 8; k < p.K; k += 64 * 8)
     {
@@ -172,7 +174,7 @@ __global__ __launch_bounds__(256) void skinny_kernel(const StackGemmParams p_in)
         {
             if (m >= p.M)
                 break;
-            const uint4 xv = *reinterpret_cast<const uint4*>(a + (int64_t) m * p.lda + k);
+            const uint4 xv = *reinterpret_cast<const uint4*>(a + arow[m] + k);
             const uint32_t xs[4] = {xv.x, xv.y, xv.z, xv.w};
 #pragma unroll
             for (int r = 0; r < SK_R; ++r)
@@ -248,6 +250,8 @@ int launch_glds_bf16(const GemmParams& g, hipStream_t stream, int m_expected = 0
         if (forced >= 0)
             pick = forced;
     }
+    if (g.act == ACT_SCALE_CAP || g.act == ACT_GELU_MUL)
+        pick = 0; // the shape whose epilogue has them
     switch (pick)
     {
     case 1: return launch_cfg<W_BF16, 4, 2, 2, 3, 1, 64, 5>(g, stream);
@@ -273,9 +277,11 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
         set_error("stack_gemm: element type %d is not served (bfloat16 or float32)", p.dtype);
         return -1;
     }
-    if (p.batch < 1 || (p.batch > 1 && p.resid) || (p.group_off && (p.resid || p.stride_a || p.stride_c)))
+    if (p.batch < 1 || (p.batch > 1 && p.resid) || (p.group_off && (p.resid || p.stride_a || p.stride_c))
+        || (p.a_rows && !p.group_off) || p.seam.n_sec < 0 || p.seam.n_sec > 2 || (p.seam.n_sec > 0 && (p.batch > 1 || p.group_off || p.resid))
+        || (p.act == ACT_GELU_MUL && (!p.seam.mul || !p.seam.mul_rows || p.group_off)))
     {
-        set_error("stack_gemm: batch %d (a batched product has no residual seam; a grouped one takes its rows from one a and one c)", p.batch);
+        set_error("stack_gemm: batch %d, act %d (a batched product has no residual seam and no output sections; a grouped one takes its rows from one a and one c)", p.batch, p.act);
         return -1;
     }
     const dim3 tiles((p.N + TN - 1) / TN, (p.M + TM - 1) / TM, p.batch);
@@ -325,6 +331,8 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
             g.gate_bias = p.gate_bias;
             g.bias = p.bias;
             g.act = p.act;
+            g.seam = p.seam;
+            g.a_rows = p.a_rows;
             if (glds)
             {
                 g.batch = p.batch;

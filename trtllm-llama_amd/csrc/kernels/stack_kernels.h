@@ -29,7 +29,10 @@ constexpr int32_t DT_BF16 = 7; // nvinfer1::DataType::kBF16
 // `batch` > 1: that many independent products of the same shape, operand b at a + b * stride_a (elements) and so on - the
 // per-head products of latent attention (one weight block per head over one slice of a shared row).
 // ---------------------------------------------------------------------------------------------
-constexpr int32_t ACT_NONE = 0, ACT_RELU2 = 1;
+// ACT_SCALE_CAP = cap * tanh(v * scale / cap) (logits), ACT_GELU_MUL = gelu_tanh(v) times an element of a table row chosen per row
+// (a per-token input gated by a projection).  Columns from seam.sec[i].col0 on may leave through output sections of their own: one
+// product over everything that reads the same input, whose columns go to different buffers, activations and types.
+constexpr int32_t ACT_NONE = GEMM_ACT_NONE, ACT_RELU2 = GEMM_ACT_RELU2, ACT_SCALE_CAP = GEMM_ACT_SCALE_CAP, ACT_GELU_MUL = GEMM_ACT_GELU_MUL;
 
 struct StackGemmParams
 {
@@ -53,6 +56,8 @@ struct StackGemmParams
     // Grouped form of a batch (a mixture of experts): device int32 [batch + 1]; product b takes rows [group_off[b], group_off[b + 1]) of
     // a and c (stride_a = stride_c = 0) and weight block b; M is the host's bound on the rows of one group.
     const int32_t* group_off = nullptr;
+    const int32_t* a_rows = nullptr; // grouped: row r of the common row range reads a's row a_rows[r] (device; no copy of the rows in group order)
+    GemmSeam seam;
     int32_t group_rows = 0; // the rows a group is expected to have (tile shapes are chosen for it), 0: M
 };
 int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream);
@@ -120,6 +125,30 @@ struct StackHyperParams
     const int32_t* rows = nullptr; // [tokens] or null
 };
 int launch_stack_hyper_norm(const StackHyperParams& p, hipStream_t stream);
+// What lands on one plain residual stream between two sublayers, and the next sublayer's norm, in one pass over a row (fp32):
+//   1. u = y, or table row ids[t] * scale (then the stream starts here: x is not read);  y_norm != null: u = u / sqrt(mean(u^2) + eps) * y_norm
+//   2. x <- x + u;  tap != null: tap = x;  add_row != null: x <- x + add_row (one row for all tokens)
+//   3. h != null: h = x / sqrt(mean(x^2) + eps) * w, or x itself where w is null (element type)
+// rows (optional gather): launch row r works on packed row rows[r], writes h row r and nothing else.
+struct StackLandParams
+{
+    int32_t dtype = DT_BF16;
+    int32_t tokens = 0, width = 0;
+    float* x = nullptr;
+    const float* y = nullptr;      // [tokens, width] or null
+    const void* table = nullptr;   // [vocab, width] of the element type or null
+    const int32_t* ids = nullptr;  // [tokens]
+    int32_t vocab = 0;
+    float scale = 1.f;
+    const float* y_norm = nullptr; // [width] or null
+    float* tap = nullptr;
+    const float* add_row = nullptr;
+    void* h = nullptr;
+    const float* w = nullptr;
+    float eps = 1e-5f;
+    const int32_t* rows = nullptr;
+};
+int launch_stack_land(const StackLandParams& p, hipStream_t stream);
 // y[t, c] = act(gu[t, c]) * gu[t, ff + c] over a [tokens, ld] projection that holds gate then up columns; act: GATE_GELU_TANH | GATE_SILU
 constexpr int32_t GATE_GELU_TANH = 0, GATE_SILU = 1;
 int launch_stack_gelu_gate(void* y, const void* gu, int32_t dtype, int32_t tokens, int32_t ff, int64_t ld, hipStream_t stream,
@@ -311,6 +340,7 @@ bool stack_ssm_serves(int32_t vdim, int32_t state, int32_t taps);
 // s + correction among the experts of the group_keep groups (of group_count equal groups of neighbours) whose largest such value is
 // largest, `top` of them; a chosen expert's weight is s * scale (without the correction, not renormalised).  The last `identity`
 // outputs are experts without weights that return h.
+// `normalize` divides the chosen scores by their sum first.  launch_stack_moe_plan = route + sort, in one launch for a few tokens.
 //   launch_stack_moe_route   -> topk_idx / topk_w [tokens, top]
 //   launch_stack_moe_sort    -> group_off [experts + 1], slot_of_pair [tokens * top] (-1: identity), a_sorted: the rows of h in
 //                               expert order, one per (token, chosen expert); the grouped products (launch_stack_gemm, group_off) run on them
@@ -333,11 +363,18 @@ struct StackMoeParams
     int32_t* group_off = nullptr;
     int32_t* slot_of_pair = nullptr;
     int32_t* pair_of_slot = nullptr;  // [tokens * top], -1 behind the last used slot
-    void* a_sorted = nullptr;         // [tokens * top, width]
+    int32_t* tok_of_slot = nullptr;   // [tokens * top] or null: the token of every used slot (grouped products read h through it: a_rows)
+    void* a_sorted = nullptr;         // [tokens * top, width]; null: no rows are copied (not with weight_input)
+    int32_t normalize = 0;            // 1: the chosen experts' scores are divided by their sum (+ 1e-20)
+    int32_t have_logits = 0;          // 1: `logits` already holds the router's logits (a projection's fp32 columns)
+    // launch_stack_moe_combine: y += the sum instead of y = it; y_el (or null) receives the resulting rows in the element type
+    int32_t accumulate = 0;
+    void* y_el = nullptr;
 };
 constexpr int32_t ROUTE_SOFTMAX = 0, ROUTE_SIGMOID = 1;
 int launch_stack_moe_route(const StackMoeParams& p, hipStream_t stream);
 int launch_stack_moe_sort(const StackMoeParams& p, hipStream_t stream);
+int launch_stack_moe_plan(const StackMoeParams& p, hipStream_t stream);
 int launch_stack_moe_combine(const StackMoeParams& p, const float* y_sorted, float* y, hipStream_t stream);
 
 // ---------------------------------------------------------------------------------------------

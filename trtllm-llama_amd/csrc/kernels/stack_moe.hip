@@ -22,6 +22,15 @@ __device__ __forceinline__ float ld_el(const void* p, int64_t i)
         return reinterpret_cast<const float*>(p)[i];
 }
 
+template <int DT>
+__device__ __forceinline__ void st_el(void* p, int64_t i, float v)
+{
+    if constexpr (DT == DT_BF16)
+        reinterpret_cast<uint16_t*>(p)[i] = f2bf(v);
+    else
+        reinterpret_cast<float*>(p)[i] = v;
+}
+
 inline int launched(const char* what)
 {
     const hipError_t e = hipGetLastError();
@@ -207,6 +216,7 @@ __device__ __forceinline__ void select_token(const StackMoeParams& p, float* zr,
         }
         __builtin_amdgcn_wave_barrier();
     }
+    float mine = 0.f, total = 0.f; // lane k keeps choice k's score; every lane their sum
     for (int k = 0; k < p.top; ++k)
     {
         float bv = -INFINITY;
@@ -223,14 +233,19 @@ __device__ __forceinline__ void select_token(const StackMoeParams& p, float* zr,
         wave_argmax(bv, bi);
         if (bi >= NE) // fewer choosable experts than `top`: the place stays empty (weight 0 on an identity)
             bi = NE - 1, bv = -INFINITY;
+        const float s = bv == -INFINITY ? 0.f : zr[bi];
+        total += s;
+        if (lane == k)
+            mine = s;
         if (lane == 0)
         {
             p.topk_idx[(int64_t) t * p.top + k] = bi;
-            p.topk_w[(int64_t) t * p.top + k] = bv == -INFINITY ? 0.f : zr[bi] * p.scale;
             cr[bi] = -INFINITY;
         }
         __builtin_amdgcn_wave_barrier();
     }
+    if (lane < p.top)
+        p.topk_w[(int64_t) t * p.top + lane] = (p.normalize ? mine / (total + 1e-20f) : mine) * p.scale;
 }
 
 // One wave per token (4 per workgroup): softmax over the logits, choice values, the kept groups, the top-k among them.
@@ -318,10 +333,9 @@ __device__ __forceinline__ void scaled_row(const StackMoeParams& p, char* dst, c
 }
 
 // One workgroup: counts per expert, offsets, a slot per pair.  Which of an expert's slots a pair gets depends on the order of the
-// atomics; a row's product does not depend on its neighbours in a tile, so the results do not.
-__global__ __launch_bounds__(1024) void moe_sort_kernel(const StackMoeParams p, int gather_row_bytes)
+// atomics; a row's product does not depend on its neighbours in a tile, so the results do not.  si: LDS, 2 * experts + 1 ints.
+__device__ __forceinline__ void sort_pairs(const StackMoeParams& p, int gather_row_bytes, int* si)
 {
-    extern __shared__ int si[];
     int* cnt = si;                  // [experts]
     int* off = cnt + p.experts;     // [experts + 1]
     const int pairs = p.tokens * p.top, tid = threadIdx.x, NT = blockDim.x;
@@ -364,6 +378,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const StackMoeParams p, 
         {
             slot = off[e] + atomicAdd(&cnt[e], 1);
             p.pair_of_slot[slot] = i;
+            if (p.tok_of_slot)
+                p.tok_of_slot[slot] = i / p.top;
         }
         p.slot_of_pair[i] = slot;
     }
@@ -388,6 +404,29 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const StackMoeParams p, 
             for (int b = lane * 2; b < gather_row_bytes; b += 64 * 2)
                 *reinterpret_cast<uint16_t*>(dst + b) = *reinterpret_cast<const uint16_t*>(src + b);
     }
+}
+
+__global__ __launch_bounds__(1024) void moe_sort_kernel(const StackMoeParams p, int gather_row_bytes)
+{
+    extern __shared__ int si[];
+    sort_pairs(p, gather_row_bytes, si);
+}
+
+// Few tokens whose logits are there already: wave t finishes token t, then the workgroup orders the pairs.
+__global__ __launch_bounds__(1024) void moe_plan_few_kernel(const StackMoeParams p, int gather_row_bytes)
+{
+    extern __shared__ float sm[];
+    const int NE = p.experts + p.identity, lane = threadIdx.x & 63, t = threadIdx.x >> 6;
+    if (t < p.tokens)
+    {
+        float* z = sm + (int64_t) t * 2 * NE;
+        for (int e = lane; e < NE; e += 64)
+            z[e] = p.logits[(int64_t) t * NE + e];
+        __builtin_amdgcn_wave_barrier();
+        select_token(p, z, z + NE, lane, t);
+    }
+    __syncthreads(); // the choices (global, this workgroup's own) are visible to all its waves
+    sort_pairs(p, gather_row_bytes, reinterpret_cast<int*>(sm));
 }
 
 // a_sorted[slot, :] = h[token of the slot's pair, :]; 16 bytes per thread where the rows allow it
@@ -427,7 +466,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const StackMoeParams p
     __syncthreads();
     for (int c = threadIdx.x; c < p.width; c += 256)
     {
-        float acc = 0.f;
+        float acc = p.accumulate ? y[(int64_t) t * p.width + c] : 0.f;
         for (int k = 0; k < p.top; ++k)
         {
             const int slot = slot_s[k];
@@ -436,6 +475,59 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const StackMoeParams p
 
         }
         y[(int64_t) t * p.width + c] = acc;
+        if (p.y_el)
+            st_el<DT>(p.y_el, (int64_t) t * p.width + c, acc);
+    }
+}
+
+// The same for rows of whole 16-byte pieces: four channels per thread, the row's channels over workgroups (blockIdx.y), every expert's
+// piece requested before the first is added.
+template <int DT, int TOP>
+__global__ __launch_bounds__(256) void moe_combine_vec_kernel(const StackMoeParams p, const float* ys, float* y)
+{
+    const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4;
+    if (c >= p.width)
+        return;
+    float4 acc = p.accumulate ? *reinterpret_cast<const float4*>(y + (int64_t) t * p.width + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int k0 = 0; k0 < p.top; k0 += TOP)
+    {
+        float4 v[TOP];
+        float w[TOP];
+#pragma unroll
+        for (int k = 0; k < TOP; ++k)
+        {
+            const bool on = k0 + k < p.top;
+            const int64_t pair = (int64_t) t * p.top + (on ? k0 + k : k0);
+            const int slot = p.slot_of_pair[pair];
+            w[k] = on ? ((p.weight_input && slot >= 0) ? 1.f : p.topk_w[pair]) : 0.f;
+            if (slot >= 0)
+                v[k] = *reinterpret_cast<const float4*>(ys + (int64_t) slot * p.width + c);
+            else
+            {
+                const int64_t o = (int64_t) t * p.width + c;
+                v[k] = make_float4(ld_el<DT>(p.h, o), ld_el<DT>(p.h, o + 1), ld_el<DT>(p.h, o + 2), ld_el<DT>(p.h, o + 3));
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < TOP; ++k)
+        {
+            if (k0 + k >= p.top)
+                break;
+            acc.x = fmaf(w[k], v[k].x, acc.x);
+            acc.y = fmaf(w[k], v[k].y, acc.y);
+            acc.z = fmaf(w[k], v[k].z, acc.z);
+            acc.w = fmaf(w[k], v[k].w, acc.w);
+        }
+    }
+    const int64_t o = (int64_t) t * p.width + c;
+    *reinterpret_cast<float4*>(y + o) = acc;
+    if (p.y_el)
+    {
+        if constexpr (DT == DT_BF16)
+            *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(p.y_el) + o)
+                = make_uint2((uint32_t) f2bf(acc.x) | ((uint32_t) f2bf(acc.y) << 16), (uint32_t) f2bf(acc.z) | ((uint32_t) f2bf(acc.w) << 16));
+        else
+            *reinterpret_cast<float4*>(reinterpret_cast<float*>(p.y_el) + o) = acc;
     }
 }
 
@@ -472,6 +564,11 @@ int launch_stack_moe_route(const StackMoeParams& p, hipStream_t stream)
         return -1;
     }
     const int NE = p.experts + p.identity;
+    if (p.have_logits)
+    {
+        hipLaunchKernelGGL(moe_select_kernel, dim3((p.tokens + 3) / 4), dim3(256), sizeof(float) * 2 * 4 * NE, stream, p, p.logits);
+        return launched("stack_moe_select");
+    }
     if (p.tokens <= FEW_TOKENS)
     {
         if (p.dtype == DT_BF16)
@@ -497,9 +594,14 @@ int launch_stack_moe_sort(const StackMoeParams& p, hipStream_t stream)
         return 0;
     if (!moe_ok(p, "stack_moe_sort"))
         return -1;
+    if (p.weight_input && !p.a_sorted)
+    {
+        set_error("stack_moe_sort: input weights need room for the scaled rows");
+        return -1;
+    }
     const size_t lds = sizeof(int) * (2 * (size_t) p.experts + 1);
-    const int row_bytes = p.width * (p.dtype == DT_BF16 ? 2 : 4);
-    const bool few = p.tokens <= FEW_TOKENS;
+    const int row_bytes = p.a_sorted ? p.width * (p.dtype == DT_BF16 ? 2 : 4) : 0;
+    const bool few = p.tokens <= FEW_TOKENS || !p.a_sorted;
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), lds, stream, p, few ? row_bytes : 0);
     const int rc = launched("stack_moe_sort");
     if (rc || few)
@@ -508,12 +610,42 @@ int launch_stack_moe_sort(const StackMoeParams& p, hipStream_t stream)
     return launched("stack_moe_gather");
 }
 
+int launch_stack_moe_plan(const StackMoeParams& p, hipStream_t stream)
+{
+    if (p.tokens <= 0)
+        return 0;
+    if (!p.have_logits || p.tokens > FEW_TOKENS)
+        return (launch_stack_moe_route(p, stream) || launch_stack_moe_sort(p, stream)) ? -1 : 0;
+    if (!moe_ok(p, "stack_moe_plan"))
+        return -1;
+    const size_t NE = (size_t) (p.experts + p.identity);
+    const size_t lds = std::max(sizeof(float) * 2 * NE * (size_t) p.tokens, sizeof(int) * (2 * (size_t) p.experts + 1));
+    if (!p.logits || (p.weight_input && !p.a_sorted) || lds > 64 * 1024)
+    {
+        set_error("stack_moe_plan: %d tokens x %d outputs, or a missing operand", p.tokens, (int) NE);
+        return -1;
+    }
+    const int row_bytes = p.a_sorted ? p.width * (p.dtype == DT_BF16 ? 2 : 4) : 0;
+    hipLaunchKernelGGL(moe_plan_few_kernel, dim3(1), dim3(1024), lds, stream, p, row_bytes);
+    return launched("stack_moe_plan");
+}
+
 int launch_stack_moe_combine(const StackMoeParams& p, const float* y_sorted, float* y, hipStream_t stream)
 {
     if (p.tokens <= 0)
         return 0;
     if (!moe_ok(p, "stack_moe_combine"))
         return -1;
+    const bool al16 = !((reinterpret_cast<uintptr_t>(y_sorted) | reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(p.y_el)) & 15);
+    if (p.width % 4 == 0 && al16)
+    {
+        const dim3 grid(p.tokens, (p.width / 4 + 255) / 256);
+        if (p.dtype == DT_BF16)
+            hipLaunchKernelGGL((moe_combine_vec_kernel<DT_BF16, 4>), grid, dim3(256), 0, stream, p, y_sorted, y);
+        else
+            hipLaunchKernelGGL((moe_combine_vec_kernel<DT_FLOAT, 4>), grid, dim3(256), 0, stream, p, y_sorted, y);
+        return launched("stack_moe_combine");
+    }
     if (p.dtype == DT_BF16)
         hipLaunchKernelGGL((moe_combine_kernel<DT_BF16>), dim3(p.tokens), dim3(256), 0, stream, p, y_sorted, y);
     else

@@ -475,12 +475,60 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const StackAttnParams 
         El<DT>::st(p.k_pool, krow + C + d, turn(p.proj, src + C, d));
 }
 
+// The same where nothing is rotated (no shared key part): the latent's norm and its two page stores, a workgroup per 8 rows of the packed
+// batch.  The value rows are channel-major inside a page, so neighbouring rows of a sequence are neighbours in memory there: the normed
+// rows pass through LDS and every thread stores one channel of up to 8 rows.
+constexpr int LS_R = 8;
+
+template <int DT>
+__global__ __launch_bounds__(256) void latent_store_kernel(const StackAttnParams p, const float* norm_w, int dkv_col)
+{
+    extern __shared__ float c_s[]; // [LS_R][C]
+    __shared__ int64_t page_row[LS_R];
+    __shared__ int page_off[LS_R];
+    const int t0 = blockIdx.x * LS_R, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, C = p.vdim;
+    const int nr = p.tokens - t0 < LS_R ? p.tokens - t0 : LS_R;
+    for (int r = wid; r < nr; r += 4)
+    {
+        const int t = t0 + r, pos = p.tok_pos[t], e = p.tok_entry[t];
+        const int blk = p.block_table[(int64_t) e * p.max_blocks + pos / p.page], off = pos % p.page;
+        const int64_t src = (int64_t) t * p.ldp + dkv_col;
+        float ss = 0.f;
+        for (int c = lane; c < C; c += 64)
+        {
+            const float x = El<DT>::ld(p.proj, src + c);
+            c_s[r * C + c] = x;
+            ss += x * x;
+        }
+        const float inv = 1.f / sqrtf(wave_sum(ss) / (float) C + p.eps);
+        const int64_t krow = ((int64_t) blk * p.page + off) * C;
+        for (int c = lane; c < C; c += 64)
+        {
+            const float x = c_s[r * C + c] * inv * norm_w[c];
+            c_s[r * C + c] = x;
+            El<DT>::st(p.k_pool, krow + c, x);
+        }
+        if (lane == 0)
+        {
+            page_row[r] = (int64_t) blk * C;
+            page_off[r] = off;
+        }
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < LS_R * C; i += 256)
+    {
+        const int c = i / LS_R, r = i % LS_R;
+        if (r < nr)
+            El<DT>::st(p.v_pool, (page_row[r] + c) * p.page + page_off[r], c_s[r * C + c]);
+    }
+}
+
 // ------------------------------------------------------------------------------------------------ attention, general form
 // One workgroup per (row, head): scores of 128 keys at a time by one thread per key, online softmax per map, P V by one thread
-// per value channel.  Any dim / vdim <= 512, both element types; the tiled kernels of stack_attn.hip take the shapes they serve.
-constexpr int AT = 128, A_CPT = 4;
+// per value channel.  Any dim, vdim up to AT * A_CPT, both element types; the tiled kernels of stack_attn.hip take the shapes they serve.
+constexpr int AT = 128;
 
-template <int DT, int MAPS>
+template <int DT, int MAPS, int A_CPT>
 __global__ __launch_bounds__(AT) void attn_general_kernel(const StackAttnParams p)
 {
     extern __shared__ float sm[];
@@ -1236,7 +1284,194 @@ void launch_hyper_vec(const StackHyperParams& p, int nt, hipStream_t stream)
         hipLaunchKernelGGL((hyper_norm_vec_kernel<DT, 8>), dim3(p.tokens), dim3(nt), 0, stream, p);
 }
 
+// One plain residual stream (StackLandParams): a row stays in registers between its loads, the norm of what lands, the addition and
+// the next sublayer's norm.  EPT float4 pieces per thread; NORM_Y: what lands is normed first.
+template <int DT>
+__device__ __forceinline__ float4 land_table4(const void* table, int64_t i)
+{
+    if constexpr (DT == DT_BF16)
+    {
+        const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const uint16_t*>(table) + i);
+        return make_float4(__builtin_bit_cast(float, u.x << 16), __builtin_bit_cast(float, u.x & 0xffff0000u), __builtin_bit_cast(float, u.y << 16),
+            __builtin_bit_cast(float, u.y & 0xffff0000u));
+    }
+    else
+        return *reinterpret_cast<const float4*>(reinterpret_cast<const float*>(table) + i);
+}
+
+template <int DT>
+__global__ __launch_bounds__(1024) void land_vec_kernel(const StackLandParams p)
+{
+    __shared__ float red[32], red2[32];
+    const int t = p.rows ? p.rows[blockIdx.x] : blockIdx.x, tid = threadIdx.x, W4 = p.width >> 2, NT = blockDim.x;
+    const int64_t row = (int64_t) t * p.width;
+    int64_t trow = 0;
+    if (p.table)
+    {
+        int id = p.ids[t];
+        id = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
+        trow = (int64_t) id * p.width;
+    }
+    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 x[HV_K], u[HV_K], yn[HV_K], ar[HV_K], wv[HV_K];
+#pragma unroll
+    for (int k = 0; k < HV_K; ++k)
+    {
+        const int c4 = tid + k * NT;
+        const bool on = c4 < W4;
+        x[k] = on && !p.table ? reinterpret_cast<const float4*>(p.x + row)[c4] : zero;
+        u[k] = zero;
+        if (on && p.table)
+        {
+            u[k] = land_table4<DT>(p.table, trow + 4 * c4);
+            u[k].x *= p.scale, u[k].y *= p.scale, u[k].z *= p.scale, u[k].w *= p.scale;
+        }
+        else if (on && p.y)
+            u[k] = reinterpret_cast<const float4*>(p.y + row)[c4];
+        yn[k] = on && p.y_norm ? reinterpret_cast<const float4*>(p.y_norm)[c4] : zero;
+        ar[k] = on && p.add_row ? reinterpret_cast<const float4*>(p.add_row)[c4] : zero;
+        wv[k] = on && p.w ? reinterpret_cast<const float4*>(p.w)[c4] : zero;
+    }
+    if (p.y_norm)
+    {
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < HV_K; ++k)
+            ss += u[k].x * u[k].x + u[k].y * u[k].y + u[k].z * u[k].z + u[k].w * u[k].w;
+        const float inv = 1.f / sqrtf(block_sum(ss, red) / (float) p.width + p.eps);
+#pragma unroll
+        for (int k = 0; k < HV_K; ++k)
+        {
+            u[k].x *= inv * yn[k].x;
+            u[k].y *= inv * yn[k].y;
+            u[k].z *= inv * yn[k].z;
+            u[k].w *= inv * yn[k].w;
+        }
+    }
+    float ss = 0.f;
+    const bool changed = p.table || p.y || p.add_row;
+#pragma unroll
+    for (int k = 0; k < HV_K; ++k)
+    {
+        const int c4 = tid + k * NT;
+        x[k].x += u[k].x, x[k].y += u[k].y, x[k].z += u[k].z, x[k].w += u[k].w;
+        if (p.tap && c4 < W4 && !p.rows)
+            reinterpret_cast<float4*>(p.tap + row)[c4] = x[k];
+        x[k].x += ar[k].x, x[k].y += ar[k].y, x[k].z += ar[k].z, x[k].w += ar[k].w;
+        if (changed && c4 < W4 && !p.rows) // a gathered launch is the stream's last reader: nothing is written back
+            reinterpret_cast<float4*>(p.x + row)[c4] = x[k];
+        ss += x[k].x * x[k].x + x[k].y * x[k].y + x[k].z * x[k].z + x[k].w * x[k].w;
+    }
+    if (!p.h)
+        return;
+    float inv = 1.f;
+    if (p.w)
+        inv = 1.f / sqrtf(block_sum(ss, red2) / (float) p.width + p.eps);
+#pragma unroll
+    for (int k = 0; k < HV_K; ++k)
+    {
+        const int c4 = tid + k * NT;
+        if (c4 >= W4)
+            continue;
+        float4 o = x[k];
+        if (p.w)
+            o = make_float4(o.x * inv * wv[k].x, o.y * inv * wv[k].y, o.z * inv * wv[k].z, o.w * inv * wv[k].w);
+        const int64_t at = (int64_t) blockIdx.x * p.width + 4 * c4;
+        if (DT == DT_BF16)
+            *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(p.h) + at)
+                = make_uint2((uint32_t) f2bf(o.x) | ((uint32_t) f2bf(o.y) << 16), (uint32_t) f2bf(o.z) | ((uint32_t) f2bf(o.w) << 16));
+        else
+            *reinterpret_cast<float4*>(reinterpret_cast<float*>(p.h) + at) = o;
+    }
+}
+
+// any width: the row in LDS
+template <int DT>
+__global__ __launch_bounds__(256) void land_kernel(const StackLandParams p)
+{
+    extern __shared__ float u_s[]; // [width]
+    __shared__ float red[32], red2[32];
+    const int t = p.rows ? p.rows[blockIdx.x] : blockIdx.x, tid = threadIdx.x, W = p.width;
+    const int64_t row = (int64_t) t * W;
+    int64_t trow = 0;
+    if (p.table)
+    {
+        int id = p.ids[t];
+        id = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
+        trow = (int64_t) id * W;
+    }
+    float ss = 0.f;
+    for (int c = tid; c < W; c += 256)
+    {
+        const float v = p.table ? El<DT>::ld(p.table, trow + c) * p.scale : (p.y ? p.y[row + c] : 0.f);
+        u_s[c] = v; // a thread reads back only what it wrote itself
+        ss += v * v;
+    }
+    float inv = 1.f;
+    if (p.y_norm)
+        inv = 1.f / sqrtf(block_sum(ss, red) / (float) W + p.eps);
+    const bool changed = p.table || p.y || p.add_row;
+    ss = 0.f;
+    for (int c = tid; c < W; c += 256)
+    {
+        float v = p.y_norm ? u_s[c] * inv * p.y_norm[c] : u_s[c];
+        if (!p.table)
+            v += p.x[row + c];
+        if (p.tap && !p.rows)
+            p.tap[row + c] = v;
+        if (p.add_row)
+            v += p.add_row[c];
+        if (changed && !p.rows)
+            p.x[row + c] = v;
+        u_s[c] = v;
+        ss += v * v;
+    }
+    if (!p.h)
+        return;
+    inv = 1.f;
+    if (p.w)
+        inv = 1.f / sqrtf(block_sum(ss, red2) / (float) W + p.eps);
+    for (int c = tid; c < W; c += 256)
+        El<DT>::st(p.h, (int64_t) blockIdx.x * W + c, p.w ? u_s[c] * inv * p.w[c] : u_s[c]);
+}
+
 } // namespace
+
+int launch_stack_land(const StackLandParams& p, hipStream_t stream)
+{
+    if (p.tokens <= 0)
+        return 0;
+    if (!known_dtype(p.dtype, "stack_land"))
+        return -1;
+    if (p.width < 1 || !p.x || (p.table && (!p.ids || p.vocab < 1 || p.y)) || (p.y_norm && !p.table && !p.y))
+    {
+        set_error("stack_land: width %d, or a missing operand", p.width);
+        return -1;
+    }
+    uintptr_t bits = 0;
+    for (const void* q : {(const void*) p.x, (const void*) p.y, p.table, (const void*) p.y_norm, (const void*) p.tap, (const void*) p.add_row, (const void*) p.h, (const void*) p.w})
+        bits |= reinterpret_cast<uintptr_t>(q);
+    if (p.width % 4 == 0 && p.width <= HV_K * 4096 && !(bits & 15))
+    {
+        const int nt = std::min(1024, (p.width / 4 + 63) / 64 * 64);
+        if (p.dtype == DT_BF16)
+            hipLaunchKernelGGL((land_vec_kernel<DT_BF16>), dim3(p.tokens), dim3(nt), 0, stream, p);
+        else
+            hipLaunchKernelGGL((land_vec_kernel<DT_FLOAT>), dim3(p.tokens), dim3(nt), 0, stream, p);
+        return launched("stack_land");
+    }
+    const size_t lds = sizeof(float) * (size_t) p.width;
+    if (lds > 60 * 1024)
+    {
+        set_error("stack_land: width %d is beyond the row it keeps in LDS", p.width);
+        return -1;
+    }
+    if (p.dtype == DT_BF16)
+        hipLaunchKernelGGL((land_kernel<DT_BF16>), dim3(p.tokens), dim3(256), lds, stream, p);
+    else
+        hipLaunchKernelGGL((land_kernel<DT_FLOAT>), dim3(p.tokens), dim3(256), lds, stream, p);
+    return launched("stack_land");
+}
 
 int launch_stack_hyper_norm(const StackHyperParams& p, hipStream_t stream)
 {
@@ -1414,6 +1649,16 @@ int launch_stack_latent_prep(const StackAttnParams& p, int32_t qk_dim, const flo
             p.dim, p.vdim, p.rot_dims, p.kv_heads, p.maps);
         return -1;
     }
+    if (p.dim == p.vdim && sizeof(float) * LS_R * (size_t) p.vdim <= 60 * 1024)
+    {
+        const size_t lds = sizeof(float) * LS_R * (size_t) p.vdim;
+        const dim3 sg((p.tokens + LS_R - 1) / LS_R);
+        if (p.dtype == DT_BF16)
+            hipLaunchKernelGGL((latent_store_kernel<DT_BF16>), sg, dim3(256), lds, stream, p, latent_norm_w, dkv_col);
+        else
+            hipLaunchKernelGGL((latent_store_kernel<DT_FLOAT>), sg, dim3(256), lds, stream, p, latent_norm_w, dkv_col);
+        return launched("stack_latent_prep (nothing rotated)");
+    }
     const dim3 grid(p.tokens, (p.heads + 1 + 3) / 4);
     if (p.dtype == DT_BF16)
         hipLaunchKernelGGL((latent_prep_kernel<DT_BF16>), grid, dim3(256), 0, stream, p, qk_dim, latent_norm_w, q_src, ldq, dkv_col);
@@ -1475,14 +1720,22 @@ int launch_stack_attention_general(const StackAttnParams& p, hipStream_t stream)
         }
         return launched("stack_attention (talking heads)");
     }
-    if (p.vdim > AT * A_CPT)
+    const size_t lds = sizeof(float) * ((size_t) p.maps * p.dim + (size_t) p.maps * AT + 32);
+    if (p.vdim > AT * 16 || lds > 60 * 1024)
     {
-        set_error("stack_attention: vdim %d is beyond the %d channels the general kernel keeps", p.vdim, AT * A_CPT);
+        set_error("stack_attention: vdim %d is beyond the %d channels the general kernel keeps (or dim %d beyond its LDS)", p.vdim, AT * 16, p.dim);
         return -1;
     }
-    const size_t lds = sizeof(float) * ((size_t) p.maps * p.dim + (size_t) p.maps * AT + 32);
     const dim3 grid(p.tokens, p.heads);
-#define TLLM_ATTN_GEN(DT, MAPS) hipLaunchKernelGGL((attn_general_kernel<DT, MAPS>), grid, dim3(AT), lds, stream, p)
+    const bool wide = p.vdim > AT * 4; // channels per thread: 4 or 16
+#define TLLM_ATTN_GEN(DT, MAPS)                                                                                     \
+    do                                                                                                               \
+    {                                                                                                                \
+        if (wide)                                                                                                    \
+            hipLaunchKernelGGL((attn_general_kernel<DT, MAPS, 16>), grid, dim3(AT), lds, stream, p);               \
+        else                                                                                                         \
+            hipLaunchKernelGGL((attn_general_kernel<DT, MAPS, 4>), grid, dim3(AT), lds, stream, p);                \
+    } while (0)
     if (p.dtype == DT_BF16)
     {
         if (p.maps == 2)

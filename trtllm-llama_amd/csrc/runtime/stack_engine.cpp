@@ -17,11 +17,21 @@
 // recurrence with skip and gate  ->  RMS norm in parts of the row;  a latent layer with a query latent projects [W_dq; W_dkv], norms
 // the query latent and expands it before the latent's pointwise part.  A routed feed-forward is  router (fp32 logits, softmax, kept
 // groups, top-k)  ->  (token, expert) pairs ordered by expert  ->  [gate_e; up_e] grouped product  ->  silu(gate) * up  ->  down_e
-// grouped product in fp32  ->  weighted sum per token (identity experts add w h).  A layer with weights_of runs on another layer's
+// grouped product in fp32  ->  weighted sum per token (identity experts add w h).  With block=parallel, residual=plain a layer run has
+// ONE norm that both sublayers read, and plain fp32 sums:
+//   P = h [Wq; Wdkv; Wg | Wshared_up | Wrouter]^T                 one product, three output sections: the mixer's columns, the shared
+//                                                                 expert's relu^2 activations (behind the context row), fp32 router logits
+//   mixer (the per-head output gate inside the attention launch)  -> ctx
+//   x += [ctx | a_shared] [Wo | Wshared_down]^T                   one product: the two sublayers' plain parts
+//   routed experts as above, read through the token of each slot; x += sum_k w_k y_k
+//   side: g = gelu(Wgate x) * e (epilogue: the layer's part of the token's side embedding); y = Wproj g
+//   x += norm(y); x += the next pass's step; h = norm1(x)         one launch, which also starts the next layer
+// A layer with weights_of runs on another layer's
 // device tensors; caches and states belong to runs.
 // The residual streams are fp32 in both element types.
 #include "../../../include/tllm_stack_api.h"
 #include "../kernels/stack_kernels.h"
+#include <algorithm>
 #include <cmath>
 #include <cstdlib>
 #include <cstring>
@@ -60,7 +70,8 @@ enum MlpKind
 {
     MLP_GELU_GATE = 0, // W_down (gelu_tanh(W_gate h) * W_up h)
     MLP_RELU2 = 1,     // W_down relu(W_up h)^2
-    MLP_MOE = 2        // routed experts W_down (silu(W_gate h) * W_up h) of size ff, the last `identity` router outputs return h
+    MLP_MOE = 2        // routed experts of size ff - W_down (silu(W_gate h) * W_up h) or W_down relu(W_up h)^2 -, the last `identity` router
+                       // outputs return h; optionally a shared expert of size shared_ff that every token uses
 };
 struct HyperW
 {
@@ -89,6 +100,7 @@ struct Layer
     int groups = 1, taps = 0, ssm_norm_groups = 1, n_conv = 0; // mamba2 (dim = state rows): B / C groups, convolution taps, parts of the output norm
     int experts = 0, identity = 0, top = 0, route_groups = 1, route_keep = 1; // moe
     double route_scale = 1;
+    int expert_relu2 = 0, route_norm = 0, shared_ff = 0, n_route = 0, n_pad = 0; // moe: experts of the relu^2 form, weights divided by their sum; columns of P
     int route_sigmoid = 0, route_weight_input = 0; // moe: sigmoid scores instead of a softmax; the weight scales the expert's input
     int mask_keep = 0, talk = 0, values_are_keys = 0, gate_wide = 0, qk_norm_weight = 0, o_bias = 0, rot_banded = 0; // attention
     int decay_rank = 0, gate_rank = 0, n_beta = 0; // delta_rule: ranks of the two low-rank projections, padded beta columns
@@ -101,6 +113,9 @@ struct Layer
           *shift = nullptr;
     void *w_a2 = nullptr, *w_g2 = nullptr; // delta_rule: the second halves of the decay's and the gate's low-rank projections
     void* w_uq = nullptr;
+    void *w_shared_up = nullptr, *w_shared_down = nullptr; // shared expert (where it is not part of w_mix / w_o)
+    void *side_gate = nullptr, *side_proj = nullptr;       // per-layer token input
+    float* side_norm = nullptr;
     HyperW hc[2];
 };
 
@@ -123,7 +138,11 @@ struct tllm_stack
     int dtype = DT_BF16, es = 2;
     int width = 0, vocab = 0, groups = 1, page = 64, blocks = 0, slots = 0, taps = 0;
     int loop_start = 0, loop_stop = 0, loop_times = 1;
-    bool sequential = false, hyper = false;
+    bool sequential = false, hyper = false, plain = false;
+    int embed_norm = 0, loop_input = 1, side_dim = 0;
+    float logit_scale = 1.f, logit_cap = 0.f;
+    void *side_embed = nullptr, *x_el = nullptr, *side_act = nullptr, *act_sh = nullptr;
+    float *embed_norm_w = nullptr, *route_z = nullptr;
     int streams = 1;
     float norm_offset = 0.f, *ones = nullptr;
     float eps = 1e-5f, emb_scale = 1.f;
@@ -148,7 +167,7 @@ struct tllm_stack
     std::vector<int32_t> last_tok;
     float *h32 = nullptr, *dl_a = nullptr, *dl_g = nullptr;
     void* pairs = nullptr; // talking heads: every query head's weights over every value head's rows, [tokens, heads * kv_heads * vdim]
-    int max_hd = 0, max_pairs = 0;
+    int max_hd = 0, max_pairs = 0, max_sh = 0;
     int max_proj = 0, max_q = 0, max_ctx = 0, max_ff = 0, max_lat = 0, max_conv = 0, max_qrank = 0, max_qfull = 0, max_top = 0, max_experts = 0, max_outputs = 0;
     int tap_tokens = 0;
 
@@ -162,11 +181,13 @@ struct tllm_stack
     }
     void free_scratch()
     {
-        void* all[] = {x, x0, o32, logits, tap, y32, h1, h2, proj, q, ctx, act, hw, lat, ints, ids_out, xbc, cq, qfull, moe_a, moe_y, moe_w, moe_i,
+        void* all[] = {x_el, side_act, act_sh, route_z, x, x0, o32, logits, tap, y32, h1, h2, proj, q, ctx, act, hw, lat, ints, ids_out, xbc, cq, qfull, moe_a, moe_y, moe_w, moe_i,
             h32, dl_a, dl_g, pairs};
         for (void* p : all)
             if (p)
                 (void) hipFree(p);
+        x_el = side_act = act_sh = nullptr;
+        route_z = nullptr;
         x = x0 = o32 = logits = tap = y32 = nullptr;
         h1 = h2 = proj = q = ctx = act = hw = lat = nullptr;
         ints = ids_out = nullptr;
@@ -315,6 +336,10 @@ int ensure_scratch(tllm_stack* s, int tokens, int want, int n_ints)
         HIP_OK(hipMalloc(&s->q, T * std::max(s->max_q, 1) * es));
         HIP_OK(hipMalloc(&s->ctx, T * std::max(s->max_ctx, 1) * es));
         HIP_OK(hipMalloc(&s->act, T * std::max(s->max_ff, 1) * es));
+        HIP_OK(hipMalloc(&s->x_el, (s->side_dim ? T * wd : 1) * es));
+        HIP_OK(hipMalloc(&s->act_sh, T * std::max(s->max_sh, 1) * es));
+        HIP_OK(hipMalloc((void**) &s->route_z, (s->plain ? T * std::max(s->max_outputs, 1) : 1) * 4));
+        HIP_OK(hipMalloc(&s->side_act, T * std::max(s->side_dim, 1) * es));
         HIP_OK(hipMalloc(&s->hw, W * wd * es));
         HIP_OK(hipMalloc((void**) &s->ints, NI * 4));
         HIP_OK(hipMalloc((void**) &s->ids_out, W * 4));
@@ -331,7 +356,7 @@ int ensure_scratch(tllm_stack* s, int tokens, int want, int n_ints)
             HIP_OK(hipMalloc(&s->moe_a, (s->max_top ? pairs * wd : 1) * es));
             HIP_OK(hipMalloc((void**) &s->moe_y, (s->max_top ? pairs * wd : 1) * 4));
             HIP_OK(hipMalloc((void**) &s->moe_w, (pairs + T * (size_t) (s->max_outputs + 1)) * 4));
-            HIP_OK(hipMalloc((void**) &s->moe_i, (3 * pairs + (size_t) s->max_experts + 1) * 4));
+            HIP_OK(hipMalloc((void**) &s->moe_i, (4 * pairs + (size_t) s->max_experts + 1) * 4));
         }
         HIP_OK(hipHostMalloc((void**) &s->pinned, NI * 4, hipHostMallocDefault));
         if (s->taps)
@@ -410,6 +435,12 @@ tllm_stack_t tllm_stack_create(const char* config_text)
     const std::string block = gets(s, "block", "parallel"), residual = gets(s, "residual", "gated");
     s->sequential = block == "sequential";
     s->hyper = residual == "hyper";
+    s->plain = residual == "plain";
+    s->embed_norm = geti(s, "embedding_norm", 0);
+    s->loop_input = geti(s, "loop_input", 1);
+    s->side_dim = geti(s, "token_side", 0);
+    s->logit_scale = (float) getd(s, "logit_scale", 1.0);
+    s->logit_cap = (float) getd(s, "logit_softcap", 0.0);
     const int L = geti(s, "num_layers", 0);
     auto fail = [&](const char* why) {
         set_error("tllm_stack_create: %s", why);
@@ -422,14 +453,22 @@ tllm_stack_t tllm_stack_create(const char* config_text)
         return fail("width must split into norm_groups equal parts");
     if (s->page < 1 || s->blocks < 1 || s->slots < 1)
         return fail("page_size, num_blocks and num_slots must be positive");
-    if ((block != "parallel" && block != "sequential") || (residual != "gated" && residual != "hyper") || s->sequential != s->hyper)
-        return fail("block=parallel goes with residual=gated, block=sequential with residual=hyper");
+    if ((block != "parallel" && block != "sequential") || (residual != "gated" && residual != "hyper" && residual != "plain") || s->sequential != s->hyper)
+        return fail("block=parallel goes with residual=gated or plain, block=sequential with residual=hyper");
+    if (!s->plain && (s->embed_norm || s->side_dim))
+        return fail("the embedding norm and the per-layer token input are built for residual=plain");
+    if (s->plain && (s->groups != 1 || s->loop_input))
+        return fail("residual=plain goes with norm_groups=1 and loop_input=0");
+    if (!s->plain && !s->loop_input)
+        return fail("loop_input=0 is built for residual=plain");
+    if (s->side_dim < 0 || s->logit_cap < 0)
+        return fail("token_side and logit_softcap must not be negative");
     if (s->streams < 1 || s->streams > 8 || (!s->hyper && s->streams != 1))
         return fail("streams: 1 to 8, more than one only with residual=hyper");
     if (s->hyper && s->loop_stop > s->loop_start)
         return fail("looped layers are built for the gated residual only");
-    if (s->pair_buckets < 0 || (s->token_shift && !s->hyper))
-        return fail("pair_buckets >= 0; the token shift is built for block=sequential");
+    if (s->pair_buckets < 0 || (s->token_shift && !s->hyper) || (s->pair_buckets && s->plain))
+        return fail("pair_buckets >= 0, not with residual=plain; the token shift is built for block=sequential");
     s->last_tok.assign((size_t) s->slots, -1);
     if (s->loop_times < 1 || s->loop_start < 0 || s->loop_stop < s->loop_start || s->loop_stop > L)
         return fail("the loop must satisfy 0 <= loop_start <= loop_stop <= num_layers, loop_times >= 1");
@@ -469,8 +508,10 @@ tllm_stack_t tllm_stack_create(const char* config_text)
         if (mlp != "gelu_gate" && mlp != "relu2" && mlp != "moe")
             return fail("a layer's mlp is gelu_gate, relu2 or moe");
         l.mlp = mlp == "relu2" ? MLP_RELU2 : (mlp == "moe" ? MLP_MOE : MLP_GELU_GATE);
-        if (l.mlp != MLP_GELU_GATE && !s->sequential)
-            return fail("the relu2 and moe feed-forwards are built for block=sequential");
+        if (l.mlp != MLP_GELU_GATE && !s->sequential && !s->plain)
+            return fail("the relu2 and moe feed-forwards are built for block=sequential and for residual=plain");
+        if (s->plain && l.ff > 0 && l.mlp != MLP_MOE)
+            return fail("residual=plain is built for the moe feed-forward");
         if ((l.kind == MIX_MAMBA2 || l.kind == MIX_DELTA || l.weights_of >= 0) && !s->sequential)
             return fail("mamba2 and delta_rule layers and shared weights are built for block=sequential");
         if (l.mlp == MLP_MOE && l.ff > 0)
@@ -484,6 +525,14 @@ tllm_stack_t tllm_stack_create(const char* config_text)
             const std::string rs = gets(s, p + "route_score", "softmax"), rw = gets(s, p + "route_weight", "output");
             if ((rs != "softmax" && rs != "sigmoid") || (rw != "output" && rw != "input"))
                 return fail("moe: route_score softmax | sigmoid, route_weight output | input");
+            const std::string ex = gets(s, p + "expert", "silu_gate");
+            if (ex != "silu_gate" && ex != "relu2")
+                return fail("moe: expert silu_gate | relu2");
+            l.expert_relu2 = ex == "relu2";
+            l.route_norm = geti(s, p + "route_norm", 0);
+            l.shared_ff = geti(s, p + "shared_ff", 0);
+            if (l.shared_ff < 0 || (l.shared_ff > 0 && !l.expert_relu2))
+                return fail("moe: the shared expert is built for the relu2 form");
             l.route_sigmoid = rs == "sigmoid";
             l.route_weight_input = rw == "input";
             const int ne = l.experts + l.identity;
@@ -494,7 +543,9 @@ tllm_stack_t tllm_stack_create(const char* config_text)
             s->max_experts = std::max(s->max_experts, l.experts);
             s->max_outputs = std::max(s->max_outputs, ne);
         }
-        l.n_rg = s->hyper ? 0 : s->width;
+        l.n_rg = (s->hyper || s->plain) ? 0 : s->width;
+        if (s->plain && l.kind != MIX_ATTENTION && l.kind != MIX_LATENT)
+            return fail("residual=plain is built for attention and latent_attention layers");
         if (l.kind == MIX_LATENT)
         {
             l.kv_rank = geti(s, p + "kv_rank", 0);
@@ -514,6 +565,8 @@ tllm_stack_t tllm_stack_create(const char* config_text)
             l.mask = mk == "window" ? MASK_WINDOW : (mk == "chunk" ? MASK_CHUNK : MASK_CAUSAL);
             l.mask_size = geti(s, p + "mask_size", 0);
             l.sink = geti(s, p + "sink", 0);
+            l.out_gate = geti(s, p + "out_gate", 0);
+            l.n_gate = l.out_gate ? l.heads : 0;
             if (l.kv_rank < 1 || l.rot_part < 0 || l.rot_dims < 0 || (l.rot_dims & 1) || l.rot_dims > l.rot_part || l.q_rank < 0)
                 return fail("latent_attention: kv_rank positive, rot_dims even and <= rot_dim");
             if (l.mask != MASK_CAUSAL && l.mask_size < 1)
@@ -636,10 +689,18 @@ tllm_stack_t tllm_stack_create(const char* config_text)
             l.n_v = l.heads * l.vdim;
         }
         l.n_mix = l.n_q + l.n_k + l.n_v + l.n_rg + l.n_gate;
+        if (s->plain)
+        {
+            // zero rows up to a multiple of 8 (rows of the element type stay 16-byte aligned); the router's columns follow the shared expert's
+            l.n_pad = (l.n_mix + 7) / 8 * 8 - l.n_mix;
+            l.n_mix += l.n_pad;
+            l.n_route = l.mlp == MLP_MOE && l.ff > 0 ? l.experts + l.identity : 0;
+        }
+        s->max_sh = std::max(s->max_sh, l.shared_ff);
         const int ff_rows = l.mlp == MLP_MOE ? l.top : 1; // a mixture's products run on one row per (token, chosen expert)
         s->max_proj = std::max(s->max_proj, std::max(l.n_mix, ff_rows * (l.mlp == MLP_RELU2 ? l.ff : 2 * l.ff) + l.n_rg));
         s->max_q = std::max(s->max_q, l.n_q);
-        s->max_ctx = std::max(s->max_ctx, l.n_ctx);
+        s->max_ctx = std::max(s->max_ctx, l.n_ctx + (s->plain ? l.shared_ff : 0));
         s->max_ff = std::max(s->max_ff, ff_rows * l.ff);
     }
     // execution order
@@ -731,6 +792,14 @@ int32_t tllm_stack_finalize(tllm_stack_t s)
         if (upload_f32(s, one.data(), one.size(), &s->ones))
             return -1;
     }
+    if (s->embed_norm && norm_vec("embed.norm", Wd, &s->embed_norm_w))
+        return -1;
+    if (s->side_dim > 0)
+    {
+        t = need(s, "side.embed", {s->vocab, (int64_t) s->side_dim * (int64_t) s->layers.size()});
+        if (!t || upload_rows(s, {t}, &s->side_embed))
+            return -1;
+    }
     if (s->pair_buckets > 0)
     {
         t = need(s, "bigram", {s->pair_buckets + 1, Wd});
@@ -756,7 +825,7 @@ int32_t tllm_stack_finalize(tllm_stack_t s)
             // the layer runs on another layer's weights: same description, same device tensors; caches and states go by run
             const Layer& src = s->layers[(size_t) l.weights_of];
             if (src.kind != l.kind || src.n_mix != l.n_mix || src.n_ctx != l.n_ctx || src.ff != l.ff || src.mlp != l.mlp || src.dim != l.dim
-                || src.heads != l.heads || src.experts != l.experts || src.identity != l.identity || src.kv_rank != l.kv_rank
+                || src.heads != l.heads || src.shared_ff != l.shared_ff || src.experts != l.experts || src.identity != l.identity || src.kv_rank != l.kv_rank
                 || src.rot_part != l.rot_part || src.taps != l.taps)
             {
                 set_error("tllm_stack_finalize: layer %d uses the weights of layer %d, but their shapes differ", (int) i, l.weights_of);
@@ -771,8 +840,16 @@ int32_t tllm_stack_finalize(tllm_stack_t s)
             return -1;
         if (s->token_shift && vec("shift", Wd, &l.shift))
             return -1;
+        if (s->side_dim > 0)
+        {
+            const HostTensor *sg = need(s, p + "side.gate", {s->side_dim, Wd}), *sp = need(s, p + "side.proj", {Wd, s->side_dim});
+            if (!sg || !sp || upload_rows(s, {sg}, &l.side_gate) || upload_rows(s, {sp}, &l.side_proj) || norm_plain(p + "side.norm", Wd, &l.side_norm))
+                return -1;
+        }
         const HostTensor* rg1 = nullptr;
-        if (!s->hyper)
+        if (s->plain)
+            ; // neither gates nor connections
+        else if (!s->hyper)
         {
             rg1 = need(s, p + "rg1", {Wd, Wd});
             if (!rg1 || vec("rg1.b", Wd, &l.rg1_b))
@@ -853,7 +930,45 @@ int32_t tllm_stack_finalize(tllm_stack_t s)
                 rows.push_back(rg1);
             if (wg)
                 rows.push_back(wg);
-            if (upload_rows(s, rows, &l.w_mix) || upload_rows(s, {wo}, &l.w_o))
+            HostTensor pad, joint;
+            const HostTensor* out_w = wo;
+            if (s->plain)
+            {
+                // everything else that reads the layer's one normed row: the shared expert's up rows and the router's
+                pad.dims = {l.n_pad, Wd};
+                pad.v.assign((size_t) pad.numel(), 0.f);
+                rows.push_back(&pad);
+                if (l.shared_ff > 0)
+                {
+                    const HostTensor *su = need(s, p + "mlp.shared.up", {l.shared_ff, Wd}), *sd = need(s, p + "mlp.shared.down", {Wd, l.shared_ff});
+                    if (!su || !sd)
+                        return -1;
+                    rows.push_back(su);
+                    if (l.kind == MIX_LATENT)
+                    {
+                        // [Wo | Wshared_down]: context and shared activations lie side by side in one row
+                        const int64_t A = l.n_ctx, B = l.shared_ff;
+                        joint.dims = {Wd, A + B};
+                        joint.v.resize((size_t) (Wd * (A + B)));
+                        for (int64_t n = 0; n < Wd; ++n)
+                        {
+                            std::copy_n(wo->v.data() + n * A, A, joint.v.data() + n * (A + B));
+                            std::copy_n(sd->v.data() + n * B, B, joint.v.data() + n * (A + B) + A);
+                        }
+                        out_w = &joint;
+                    }
+                    else if (upload_rows(s, {sd}, &l.w_shared_down))
+                        return -1;
+                }
+                if (l.n_route > 0)
+                {
+                    const HostTensor* rw = need(s, p + "mlp.router", {l.n_route, Wd});
+                    if (!rw)
+                        return -1;
+                    rows.push_back(rw);
+                }
+            }
+            if (upload_rows(s, rows, &l.w_mix) || upload_rows(s, {out_w}, &l.w_o))
                 return -1;
         }
         if (l.kind == MIX_ATTENTION || l.kind == MIX_LATENT)
@@ -966,18 +1081,26 @@ int32_t tllm_stack_finalize(tllm_stack_t s)
             // experts stacked: [gate_e; up_e] rows per expert, then the down matrices; router and correction stay fp32
             const int ne = l.experts + l.identity;
             const HostTensor* rw = need(s, p + "mlp.router", {ne, Wd});
-            if (norm_vec(p + "norm2", Wd, &l.norm2) || !rw || upload_f32(s, rw->v.data(), rw->v.size(), &l.router_w))
+            if (!rw || (!s->plain && (norm_vec(p + "norm2", Wd, &l.norm2) || upload_f32(s, rw->v.data(), rw->v.size(), &l.router_w))))
                 return -1;
+            if (!s->plain && l.shared_ff > 0)
+            {
+                const HostTensor *su = need(s, p + "mlp.shared.up", {l.shared_ff, Wd}), *sd = need(s, p + "mlp.shared.down", {Wd, l.shared_ff});
+                if (!su || !sd || upload_rows(s, {su}, &l.w_shared_up) || upload_rows(s, {sd}, &l.w_shared_down))
+                    return -1;
+            }
             if (s->host.count(p + "mlp.correction") && vec("mlp.correction", ne, &l.correction))
                 return -1;
             std::vector<const HostTensor*> gu, dn;
             for (int e = 0; e < l.experts; ++e)
             {
                 const std::string ep = p + "mlp.e" + std::to_string(e) + ".";
-                const HostTensor *g = need(s, ep + "gate", {l.ff, Wd}), *u = need(s, ep + "up", {l.ff, Wd}), *d = need(s, ep + "down", {Wd, l.ff});
-                if (!g || !u || !d)
+                const HostTensor *g = l.expert_relu2 ? nullptr : need(s, ep + "gate", {l.ff, Wd}), *u = need(s, ep + "up", {l.ff, Wd}),
+                                 *d = need(s, ep + "down", {Wd, l.ff});
+                if ((!g && !l.expert_relu2) || !u || !d)
                     return -1;
-                gu.push_back(g);
+                if (g)
+                    gu.push_back(g);
                 gu.push_back(u);
                 dn.push_back(d);
             }
@@ -1173,7 +1296,8 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
     const int Wd = s->width;
     const bool looped = s->loop_stop > s->loop_start;
     const int64_t stream_stride = (int64_t) T * Wd;
-    if (launch_stack_embed(s->x, looped && s->loop_times > 1 ? s->x0 : nullptr, d_tok, s->embed, s->dtype, T, Wd, s->vocab, s->emb_scale, stream,
+    if (!s->plain // (a plain residual starts in the launch of its first norm)
+        && launch_stack_embed(s->x, looped && s->loop_times > 1 ? s->x0 : nullptr, d_tok, s->embed, s->dtype, T, Wd, s->vocab, s->emb_scale, stream,
             s->streams, stream_stride))
         return -1;
     if (s->pair_buckets > 0
@@ -1182,8 +1306,9 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         return -1;
     s->tap_tokens = T;
 
-    // P1 = h1 W_mix^T, then the mixer: its context rows land in s->ctx
+    // P1 = h1 W_mix^T, then the mixer: its context rows land in s->ctx, ld_ctx elements apart
     auto run_mixer = [&](const Layer& l, const Run& r) -> int {
+        const int64_t ld_ctx = l.n_ctx + (s->plain && l.kind == MIX_LATENT ? l.shared_ff : 0);
         StackGemmParams g;
         g.dtype = s->dtype;
         g.M = T;
@@ -1194,6 +1319,24 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         g.w = l.w_mix;
         g.c = s->proj;
         g.ldc = l.n_mix;
+        if (s->plain && l.shared_ff > 0)
+        {
+            GemmSection& sec = g.seam.sec[g.seam.n_sec++];
+            sec.col0 = g.N;
+            sec.c = l.kind == MIX_LATENT ? (char*) s->ctx + (size_t) l.n_ctx * s->es : (char*) s->act_sh;
+            sec.ldc = l.kind == MIX_LATENT ? ld_ctx : l.shared_ff;
+            sec.act = ACT_RELU2;
+            g.N += l.shared_ff;
+        }
+        if (l.n_route > 0)
+        {
+            GemmSection& sec = g.seam.sec[g.seam.n_sec++];
+            sec.col0 = g.N;
+            sec.c = s->route_z;
+            sec.ldc = l.n_route;
+            sec.f32 = 1;
+            g.N += l.n_route;
+        }
         if (launch_stack_gemm(g, stream))
             return -1;
         if (l.kind == MIX_DELTA)
@@ -1366,6 +1509,12 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
             a.mask = l.mask;
             a.mask_size = l.mask_size;
             a.sink = l.sinkv;
+            if (l.n_gate)
+            {
+                // the gate scales a head's whole row, so it commutes with the expansion behind the attention
+                a.out_gate = (const char*) s->proj + (size_t) (l.n_q + l.n_k + l.n_v + l.n_rg) * s->es;
+                a.ld_gate = l.n_mix;
+            }
             a.out = s->lat;
             const void* q_src = s->proj;
             int64_t ldq = l.n_mix;
@@ -1416,7 +1565,7 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
             ve.lda = (int64_t) H * C;
             ve.w = l.w_uv;
             ve.c = s->ctx;
-            ve.ldc = l.n_ctx;
+            ve.ldc = ld_ctx;
             ve.batch = H;
             ve.stride_a = C;
             ve.stride_w = (int64_t) l.vdim * C;
@@ -1460,6 +1609,109 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         return (launch_stack_rope_kv(a, stream) || launch_stack_attention(a, stream)) ? -1 : 0;
     };
 
+    // the routed feed-forward on h1: y32 = its output, or (accumulate) x += it, x_el = the resulting rows in the element type.  With
+    // residual=plain the router's logits are there already.
+    auto run_moe = [&](const Layer& l, float* y, bool accumulate, void* y_el) -> int {
+        const size_t pairs = (size_t) T * l.top;
+        StackMoeParams mp;
+        mp.dtype = s->dtype;
+        mp.tokens = T;
+        mp.width = Wd;
+        mp.experts = l.experts;
+        mp.identity = l.identity;
+        mp.top = l.top;
+        mp.group_count = l.route_groups;
+        mp.group_keep = l.route_keep;
+        mp.scale = (float) l.route_scale;
+        mp.score = l.route_sigmoid ? ROUTE_SIGMOID : ROUTE_SOFTMAX;
+        mp.weight_input = l.route_weight_input;
+        mp.normalize = l.route_norm;
+        mp.h = s->h1;
+        mp.router_w = l.router_w;
+        mp.correction = l.correction;
+        mp.topk_idx = s->moe_i;
+        mp.slot_of_pair = s->moe_i + pairs;
+        mp.pair_of_slot = s->moe_i + 2 * pairs;
+        mp.tok_of_slot = s->moe_i + 3 * pairs;
+        mp.group_off = s->moe_i + 4 * pairs;
+        mp.topk_w = s->moe_w;
+        mp.logits = s->plain ? s->route_z : s->moe_w + pairs;
+        mp.have_logits = s->plain ? 1 : 0;
+        mp.a_sorted = l.route_weight_input ? s->moe_a : nullptr; // otherwise the products read h1 through the slots' tokens
+        mp.accumulate = accumulate ? 1 : 0;
+        mp.y_el = y_el;
+        if (launch_stack_moe_plan(mp, stream))
+            return -1;
+        // per expert: [gate; up] on its rows, silu(gate) * up (or relu(up)^2), down in fp32; an expert's rows are at most one per token
+        const int up_cols = l.expert_relu2 ? l.ff : 2 * l.ff;
+        StackGemmParams u;
+        u.dtype = s->dtype;
+        u.M = T;
+        u.N = up_cols;
+        u.K = Wd;
+        u.a = mp.a_sorted ? s->moe_a : s->h1;
+        u.a_rows = mp.a_sorted ? nullptr : mp.tok_of_slot;
+        u.lda = Wd;
+        u.w = l.w_gu;
+        u.c = l.expert_relu2 ? s->act : s->proj;
+        u.ldc = up_cols;
+        u.act = l.expert_relu2 ? ACT_RELU2 : ACT_NONE;
+        u.batch = l.experts;
+        u.stride_w = (int64_t) up_cols * Wd;
+        u.group_off = mp.group_off;
+        u.group_rows = (int) std::min<int64_t>(T, (pairs + l.experts - 1) / l.experts);
+        if (launch_stack_gemm(u, stream)
+            || (!l.expert_relu2 && launch_stack_gelu_gate(s->act, s->proj, s->dtype, (int) pairs, l.ff, u.N, stream, GATE_SILU)))
+            return -1;
+        StackGemmParams dn;
+        dn.dtype = s->dtype;
+        dn.out_f32 = 1;
+        dn.M = T;
+        dn.N = Wd;
+        dn.K = l.ff;
+        dn.a = s->act;
+        dn.lda = l.ff;
+        dn.w = l.w_down;
+        dn.c = s->moe_y;
+        dn.ldc = Wd;
+        dn.batch = l.experts;
+        dn.stride_w = (int64_t) Wd * l.ff;
+        dn.group_off = mp.group_off;
+        dn.group_rows = u.group_rows;
+        return (launch_stack_gemm(dn, stream) || launch_stack_moe_combine(mp, s->moe_y, y, stream)) ? -1 : 0;
+    };
+
+    // residual=plain: what the last layer left to land (its token input's result in y32) and the next norm, in one launch
+    const float* land_norm = nullptr; // weight of the norm on y32; null: nothing to land
+    auto land = [&](void* h, const float* w, const float* add_row, const int32_t* rows, int n, float* tap, bool start) -> int {
+        StackLandParams lp;
+        lp.dtype = s->dtype;
+        lp.tokens = n;
+        lp.width = Wd;
+        lp.x = s->x;
+        if (start)
+        {
+            lp.table = s->embed;
+            lp.ids = d_tok;
+            lp.vocab = s->vocab;
+            lp.scale = s->emb_scale;
+            lp.y_norm = s->embed_norm_w;
+        }
+        else if (land_norm)
+        {
+            lp.y = s->y32;
+            lp.y_norm = land_norm;
+        }
+        lp.tap = tap;
+        lp.add_row = add_row;
+        lp.h = h;
+        lp.w = w;
+        lp.eps = s->eps;
+        lp.rows = rows;
+        land_norm = nullptr;
+        return launch_stack_land(lp, stream);
+    };
+
     // residual=hyper: the sublayer result in y32 that has not yet been folded into the streams, and the launch that folds it,
     // combines the streams for the next reader and norms the combination
     const HyperW* pending = nullptr;
@@ -1491,6 +1743,72 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
     {
         const Run& r = s->runs[ri];
         const Layer& l = s->layers[r.layer];
+        if (s->plain)
+        {
+            if (land(s->h1, l.norm1, r.enters_pass ? s->loop_step + (size_t) r.pass * Wd : nullptr, nullptr, T,
+                    s->taps && ri > 0 ? s->tap + (ri - 1) * (size_t) T * Wd : nullptr, ri == 0))
+                return -1;
+            if (run_mixer(l, r))
+                return -1;
+            const bool joint = l.kind == MIX_LATENT && l.shared_ff > 0;
+            StackGemmParams o; // x += [ctx | a_shared] [Wo | Wshared_down]^T
+            o.dtype = s->dtype;
+            o.M = T;
+            o.N = Wd;
+            o.K = l.n_ctx + (joint ? l.shared_ff : 0);
+            o.a = s->ctx;
+            o.lda = o.K;
+            o.w = l.w_o;
+            o.resid = s->x;
+            o.ldr = Wd;
+            if (launch_stack_gemm(o, stream))
+                return -1;
+            if (l.shared_ff > 0 && !joint)
+            {
+                o.K = l.shared_ff;
+                o.a = s->act_sh;
+                o.lda = o.K;
+                o.w = l.w_shared_down;
+                if (launch_stack_gemm(o, stream))
+                    return -1;
+            }
+            if (l.ff > 0 && run_moe(l, s->x, true, s->side_dim ? s->x_el : nullptr))
+                return -1;
+            if (s->side_dim > 0)
+            {
+                if (l.ff == 0 && land(s->x_el, nullptr, nullptr, nullptr, T, nullptr, false))
+                    return -1;
+                StackGemmParams sg; // g = gelu(Wgate x) * the layer's part of the token's side embedding
+                sg.dtype = s->dtype;
+                sg.M = T;
+                sg.N = s->side_dim;
+                sg.K = Wd;
+                sg.a = s->x_el;
+                sg.lda = Wd;
+                sg.w = l.side_gate;
+                sg.c = s->side_act;
+                sg.ldc = s->side_dim;
+                sg.act = ACT_GELU_MUL;
+                sg.seam.mul = (const char*) s->side_embed + (size_t) r.layer * s->side_dim * s->es;
+                sg.seam.mul_rows = d_tok;
+                sg.seam.ld_mul = (int64_t) s->side_dim * (int64_t) s->layers.size();
+                StackGemmParams sp;
+                sp.dtype = s->dtype;
+                sp.out_f32 = 1;
+                sp.M = T;
+                sp.N = Wd;
+                sp.K = s->side_dim;
+                sp.a = s->side_act;
+                sp.lda = s->side_dim;
+                sp.w = l.side_proj;
+                sp.c = s->y32;
+                sp.ldc = Wd;
+                if (launch_stack_gemm(sg, stream) || launch_stack_gemm(sp, stream))
+                    return -1;
+                land_norm = l.side_norm;
+            }
+            continue;
+        }
         if (s->hyper)
         {
             if (s->token_shift)
@@ -1547,60 +1865,28 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
                 const void* act = s->act;
                 if (l.mlp == MLP_MOE)
                 {
-                    const size_t pairs = (size_t) T * l.top;
-                    StackMoeParams mp;
-                    mp.dtype = s->dtype;
-                    mp.tokens = T;
-                    mp.width = Wd;
-                    mp.experts = l.experts;
-                    mp.identity = l.identity;
-                    mp.top = l.top;
-                    mp.group_count = l.route_groups;
-                    mp.group_keep = l.route_keep;
-                    mp.scale = (float) l.route_scale;
-                    mp.score = l.route_sigmoid ? ROUTE_SIGMOID : ROUTE_SOFTMAX;
-                    mp.weight_input = l.route_weight_input;
-                    mp.h = s->h1;
-                    mp.router_w = l.router_w;
-                    mp.correction = l.correction;
-                    mp.topk_idx = s->moe_i;
-                    mp.slot_of_pair = s->moe_i + pairs;
-                    mp.pair_of_slot = s->moe_i + 2 * pairs;
-                    mp.group_off = s->moe_i + 3 * pairs;
-                    mp.topk_w = s->moe_w;
-                    mp.logits = s->moe_w + pairs;
-                    mp.a_sorted = s->moe_a;
-                    if (launch_stack_moe_route(mp, stream) || launch_stack_moe_sort(mp, stream))
-                        return -1;
-                    // per expert: [gate; up] on its rows, silu(gate) * up, down in fp32; an expert's rows are at most one per token
-                    u.M = T;
-                    u.N = 2 * l.ff;
-                    u.a = s->moe_a;
-                    u.c = s->proj;
-                    u.ldc = u.N;
-                    u.batch = l.experts;
-                    u.stride_w = (int64_t) 2 * l.ff * Wd;
-                    u.group_off = mp.group_off;
-                    u.group_rows = (int) std::min<int64_t>(T, (pairs + l.experts - 1) / l.experts);
-                    if (launch_stack_gemm(u, stream)
-                        || launch_stack_gelu_gate(s->act, s->proj, s->dtype, (int) pairs, l.ff, u.N, stream, GATE_SILU))
-                        return -1;
-                    StackGemmParams dn;
-                    dn.dtype = s->dtype;
-                    dn.out_f32 = 1;
-                    dn.M = T;
-                    dn.N = Wd;
-                    dn.K = l.ff;
-                    dn.a = s->act;
-                    dn.lda = l.ff;
-                    dn.w = l.w_down;
-                    dn.c = s->moe_y;
-                    dn.ldc = Wd;
-                    dn.batch = l.experts;
-                    dn.stride_w = (int64_t) Wd * l.ff;
-                    dn.group_off = mp.group_off;
-                    dn.group_rows = u.group_rows;
-                    if (launch_stack_gemm(dn, stream) || launch_stack_moe_combine(mp, s->moe_y, s->y32, stream))
+                    if (l.shared_ff > 0)
+                    {
+                        u.N = l.shared_ff;
+                        u.c = s->act_sh;
+                        u.ldc = l.shared_ff;
+                        u.act = ACT_RELU2;
+                        StackGemmParams sd;
+                        sd.dtype = s->dtype;
+                        sd.out_f32 = 1;
+                        sd.M = T;
+                        sd.N = Wd;
+                        sd.K = l.shared_ff;
+                        sd.a = s->act_sh;
+                        sd.lda = l.shared_ff;
+                        sd.w = l.w_shared_down;
+                        sd.c = s->y32;
+                        sd.ldc = Wd;
+                        u.w = l.w_shared_up;
+                        if (launch_stack_gemm(u, stream) || launch_stack_gemm(sd, stream))
+                            return -1;
+                    }
+                    if (run_moe(l, s->y32, l.shared_ff > 0, nullptr))
                         return -1;
                     pending = &l.hc[1];
                     if (s->taps && hyper(nullptr, nullptr, nullptr, s->tap + ri * (size_t) T * Wd))
@@ -1705,9 +1991,17 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         if (s->taps)
             HIP_OK(hipMemcpyAsync(s->tap + ri * (size_t) T * Wd, s->x, (size_t) T * Wd * 4, hipMemcpyDeviceToDevice, stream));
     }
+    if (s->plain && s->taps && land(nullptr, nullptr, nullptr, nullptr, T, s->tap + (s->runs.size() - 1) * (size_t) T * Wd, false))
+        return -1;
     if (NW > 0)
     {
-        if (s->hyper)
+        if (s->plain)
+        {
+            // the output norm, on the wanted rows only; what the last layer left lands in the same launch
+            if (land(s->hw, s->final_norm, nullptr, d_want, NW, nullptr, false))
+                return -1;
+        }
+        else if (s->hyper)
         {
             // the output norm reads the sum of the streams; the last sublayer lands in the same launch, on the wanted rows only
             StackHyperParams hp;
@@ -1743,6 +2037,12 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         hd.w = s->head;
         hd.c = s->logits;
         hd.ldc = s->vocab;
+        if (s->logit_scale != 1.f || s->logit_cap > 0.f)
+        {
+            hd.act = ACT_SCALE_CAP;
+            hd.seam.act_scale = s->logit_scale;
+            hd.seam.act_cap = s->logit_cap;
+        }
         if (launch_stack_gemm(hd, stream))
             return -1;
         if (next_ids_out && launch_argmax(s->ids_out, s->logits, NW, s->vocab, stream))
@@ -1791,13 +2091,15 @@ int64_t tllm_stack_step_bytes(tllm_stack_t s, int32_t n_tokens, int64_t context_
     for (const Run& r : s->runs)
     {
         const Layer& l = s->layers[r.layer];
-        int64_t ff_rows = l.ff > 0 ? (l.mlp == MLP_RELU2 ? 2 : 3) * (int64_t) l.ff + l.n_rg : 0;
+        int64_t ff_rows = l.ff > 0 ? (l.mlp == MLP_RELU2 || l.expert_relu2 ? 2 : 3) * (int64_t) l.ff + l.n_rg : 0;
         if (l.ff > 0 && l.mlp == MLP_MOE)
         {
             // the experts that the step's tokens can reach at most, and the fp32 router
             ff_rows *= std::min<int64_t>(l.experts, (int64_t) n_tokens * l.top);
-            bytes += (int64_t) (l.experts + l.identity) * s->width * 4;
+            bytes += (int64_t) (l.experts + l.identity) * s->width * (s->plain ? s->es : 4);
+            ff_rows += 2 * (int64_t) l.shared_ff;
         }
+        bytes += 2 * (int64_t) s->side_dim * s->width * s->es + (int64_t) n_tokens * s->side_dim * s->es; // the token input
         bytes += ((int64_t) l.n_mix + l.n_ctx + ff_rows) * s->width * s->es;
         if (l.kind == MIX_LATENT && l.q_rank > 0)
             bytes += (int64_t) l.heads * (l.dim + l.rot_part) * l.q_rank * s->es;

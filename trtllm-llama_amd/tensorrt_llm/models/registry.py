@@ -8,6 +8,7 @@ import os
 from .llama.model import LLaMAForCausalLM
 from .narurax.model import NaruraxForCausalLM
 from .rofozen.model import RofozenForCausalLM
+from .sodudra.model import SodudraForCausalLM
 from .tolenex.model import TolenexForCausalLM
 from .vetipel.model import VetipelForCausalLM
 
@@ -16,6 +17,7 @@ MODEL_REGISTRY = {
     'LLaMAForCausalLM': LLaMAForCausalLM,
     'Narurax': NaruraxForCausalLM,
     'Rofozen': RofozenForCausalLM,
+    'Sodudra': SodudraForCausalLM,
     'Tolenex': TolenexForCausalLM,
     'Vetipel': VetipelForCausalLM,
 }
