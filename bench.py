@@ -62,7 +62,7 @@ def parse():
     ap.add_argument('--parity-prompts', type=int, default=8, help='seeded prompts of the accuracy report')
     ap.add_argument('--cpu-tokens', type=int, default=0, help='CPU-baseline decode steps (0 = sized to ~20 s)')
     ap.add_argument('--cpu-threads', type=int, default=0)
-    ap.add_argument('--design', default='llama', choices=['llama', 'tolenex', 'vetipel', 'rofozen', 'narurax'],
+    ap.add_argument('--design', default='llama', choices=['llama', 'tolenex', 'vetipel', 'rofozen', 'narurax', 'sodudra'],
                     help="tolenex: a side report instead of the headline workload - prefill and decode throughput of the Tolenex design "
                          "(bfloat16, ragged stack engine) at layer sizes of real models, beside LLaMA fp16 at equal size; "
                          "vetipel: the same report for the Vetipel design, beside Tolenex (the closest model: same engine, bfloat16) and "
@@ -71,7 +71,9 @@ def parse():
     # Tolenex, the closest model: a recurrent / attention hybrid on the same engine in bfloat16, and Vetipel and LLaMA fp16 at equal size;
     # narurax: the same report for the Narurax design - attention with kept first tokens, sinks and head-mixed weights, a per-channel gated
     # delta rule, token shift, input-weighted sigmoid routing - beside Rofozen, the closest model: a recurrent / attention hybrid with
-    # routed experts on the same engine in bfloat16)
+    # routed experts on the same engine in bfloat16;
+    # sodudra: the same report for the Sodudra design - latent attention without positions, relu^2 experts with a shared one, per-layer
+    # token input, a looped layer - beside Rofozen, the closest model: latent attention and routed experts on the same engine)
     ap.add_argument('--design-sizes', default='2048,4096', help='--design tolenex: comma list of model widths')
     ap.add_argument('--design-no-llama', action='store_true', help='--design tolenex: skip the LLaMA side (kernel traces of the new design alone)')
     ap.add_argument('--design-alone', action='store_true', help='--design vetipel: time that design only (kernel traces without its neighbours)')
@@ -654,6 +656,23 @@ def narurax_config(width, layers, vocab=32000):
             'layers': [{'type': kinds[i % 4][0], 'mixer': dict(kinds[i % 4][1]), 'mlp': dict(moe)} for i in range(layers)]}
 
 
+def sodudra_config(width, layers, vocab=32000):
+    """A Sodudra configuration with the layer sizes of a LLaMA-like model of this width: heads of 128 query / key and value dimensions
+    over a latent of 256, every feed-forward routing 4 of 32 relu^2 experts of a quarter of 2.6875 x width beside a shared expert of
+    twice that size, a token input of 256 channels per layer.  `layers` layer runs: the second layer runs twice, as Rofozen's last
+    layer runs on its second layer's weights."""
+    heads = width // 128
+    eff = -(-int(width * 2.6875 / 4) // 64) * 64
+    lat = {'heads': heads, 'dim': 128, 'vdim': 128, 'kv_rank': 256, 'scale': 128 ** -0.5}
+    moe = {'kind': 'moe', 'expert': {'ff': eff}, 'router': {'experts': 32, 'top': 4}, 'shared': {'ff': 2 * eff}}
+    cfg = {'architecture': 'Sodudra', 'vocab': vocab, 'width': width, 'norm': {'eps': 1e-6}, 'logit_scale': 0.5, 'logit_softcap': 20.0,
+           'token_side': {'dim': 256},
+           'layers': [{'type': 'latent_attention', 'mixer': dict(lat), 'mlp': dict(moe)} for _ in range(max(layers - 1, 1))]}
+    if layers > 2:
+        cfg['loop'] = {'start': 1, 'stop': 2, 'times': 2}
+    return cfg
+
+
 def time_stack_model(torch, model, vocab, S, K, W, tag, row):
     """Prefill (one step of S prompt tokens) and decode (single tokens at context S, 1 and 4 sequences per step) of a stack-engine
     model in bfloat16 through RaggedGenerationSession.step; wall clock around synchronised calls."""
@@ -708,11 +727,19 @@ def tolenex_report(torch, args, dev):
                 rows.append({k: (round(v, 3) if isinstance(v, float) else v) for k, v in row.items()})
                 print(f'[bench] {rows[-1]}', file=sys.stderr, flush=True)
                 continue
-        if args.design in ('rofozen', 'narurax'):
+        if args.design == 'sodudra':
+            from tensorrt_llm.models import SodudraForCausalLM
+            scfg = sodudra_config(width, L)
+            time_stack_model(torch, SodudraForCausalLM.from_random(scfg, seed=1), scfg['vocab'], S, K, W, 'sodudra', row)
+            if args.design_alone:
+                rows.append({k: (round(v, 3) if isinstance(v, float) else v) for k, v in row.items()})
+                print(f'[bench] {rows[-1]}', file=sys.stderr, flush=True)
+                continue
+        if args.design in ('rofozen', 'narurax', 'sodudra'):
             from tensorrt_llm.models import RofozenForCausalLM
             rcfg = rofozen_config(width, L)
             time_stack_model(torch, RofozenForCausalLM.from_random(rcfg, seed=1), rcfg['vocab'], S, K, W, 'rofozen', row)
-            if args.design_alone or args.design == 'narurax':
+            if args.design_alone or args.design in ('narurax', 'sodudra'):
                 rows.append({k: (round(v, 3) if isinstance(v, float) else v) for k, v in row.items()})
                 print(f'[bench] {rows[-1]}', file=sys.stderr, flush=True)
                 continue
@@ -801,7 +828,7 @@ def main():
         local = 0
     torch.cuda.set_device(local)
     dev = torch.device('cuda', local)
-    if args.design in ('tolenex', 'vetipel', 'rofozen', 'narurax'):
+    if args.design in ('tolenex', 'vetipel', 'rofozen', 'narurax', 'sodudra'):
         if world != 1:
             raise SystemExit(f'--design {args.design} is a one-GPU report')
         return tolenex_report(torch, args, dev)
