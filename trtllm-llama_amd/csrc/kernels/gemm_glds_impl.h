@@ -441,7 +441,7 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
                     if constexpr (WT == W_BF16)
                     {
                         if (relu2_col[j])
-                            v = seam_relu2(bf2f(f2bf(v)));
+                            v = seam_relu2(v);
                     }
                     *reinterpret_cast<uint16_t*>(scr + rr * PITCH + (j * 32 + (lane & 31)) * 2) = WT == W_BF16 ? f2bf(v) : f2h(v);
                 }

@@ -61,7 +61,7 @@ __device__ __forceinline__ void seam_store(const GemmSeam& s, const SeamOut& o, 
     if (o.act != GEMM_ACT_NONE)
     {
         if (o.act == GEMM_ACT_RELU2)
-            v = seam_relu2(o.f32 ? v : bf2f(f2bf(v))); // the projection's value in its element type, then its activation
+            v = seam_relu2(v);
         else if (!ALL_ACTS)
             ;
         else if (o.act == GEMM_ACT_SCALE_CAP)
@@ -77,9 +77,8 @@ __device__ __forceinline__ void seam_store(const GemmSeam& s, const SeamOut& o, 
         }
         else
         {
-            const float z = o.f32 ? v : bf2f(f2bf(v));
-            const float u = 2.f * 0.7978845608028654f * (z + 0.044715f * z * z * z); // (1 + tanh(u / 2)) / 2 = 1 / (1 + e^-u)
-            v = z / (1.f + (EL_F32 ? expf(-u) : __expf(-u))) * seam_ld<EL_F32>(s.mul, (int64_t) s.mul_rows[row] * s.ld_mul + col);
+            const float u = 2.f * 0.7978845608028654f * (v + 0.044715f * v * v * v); // (1 + tanh(u / 2)) / 2 = 1 / (1 + e^-u)
+            v = v / (1.f + (EL_F32 ? expf(-u) : __expf(-u))) * seam_ld<EL_F32>(s.mul, (int64_t) s.mul_rows[row] * s.ld_mul + col);
         }
     }
     const int64_t at = (int64_t) row * o.ldc + col;

@@ -329,9 +329,9 @@ int launch_context_attention(const ContextAttnParams& p, hipStream_t stream);
 // ---------------------------------------------------------------------------------------------
 // What a bfloat16 product of the stack engine may do with its result besides a plain store (gemm_seam.h applies it).
 constexpr int32_t GEMM_ACT_NONE = 0;
-constexpr int32_t GEMM_ACT_RELU2 = 1;     // max(v, 0)^2 of the value rounded to the output type
+constexpr int32_t GEMM_ACT_RELU2 = 1;     // max(v, 0)^2
 constexpr int32_t GEMM_ACT_SCALE_CAP = 2; // v * act_scale, then act_cap * tanh(v / act_cap) where act_cap > 0
-constexpr int32_t GEMM_ACT_GELU_MUL = 3;  // gelu_tanh(v of the output type) * mul[mul_rows[m], n]
+constexpr int32_t GEMM_ACT_GELU_MUL = 3;  // gelu_tanh(v) * mul[mul_rows[m], n]
 struct GemmSection
 {
     int32_t col0 = 0;  // first column of the section (the section before it ends here)

@@ -25,7 +25,7 @@ constexpr int32_t DT_BF16 = 7; // nvinfer1::DataType::kBF16
 //   dtype DT_FLOAT: fp32 FMA tiles (stack_gemm.hip).
 // Epilogue, when `resid` is set: resid[m, n] += sigmoid(gate[m, n] + gate_bias[n]) * C[m, n]  (fp32 residual stream, the
 // sublayer's gate taken from another projection's columns); nothing is written to `c` then.  Otherwise `bias` (fp32 [N]) is added
-// to the accumulator and `act` is applied to the value rounded to the element type: ACT_RELU2 = max(v, 0)^2.
+// to the accumulator and `act` is applied in fp32 ahead of the one rounding to the element type: ACT_RELU2 = max(v, 0)^2.
 // `batch` > 1: that many independent products of the same shape, operand b at a + b * stride_a (elements) and so on - the
 // per-head products of latent attention (one weight block per head over one slice of a shared row).
 // ---------------------------------------------------------------------------------------------
