@@ -6,6 +6,7 @@
 #include "gemm_seam.h"
 #include "kernels.h"
 #include "launch_util.h"
+#include <algorithm>
 
 namespace tllm
 {
@@ -61,6 +62,56 @@ __device__ __forceinline__ void wait_vmcnt()
     asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
 }
 
+// Which tile of which group workgroup `wg` of a grouped launch takes.  The groups' row counts are the device's (group_off), so every
+// wave forms the running sum of their tile counts itself (64 groups per step).  The tiles that exist are numbered group by group, inside
+// a group column panel by column panel, and each XCD (workgroups go round them) takes a contiguous range of the numbers: the row tiles
+// that share a weight panel run side by side on one L2.  group < 0: no tile is left.
+struct GroupTile
+{
+    int group, tile;
+};
+template <int BM>
+__device__ __forceinline__ GroupTile group_tile(const GemmParams& p, int tiles_n, int wg)
+{
+    const int lane = threadIdx.x & 63;
+    auto tiles_of = [&](int g) { return g < p.batch ? (p.group_off[g + 1] - p.group_off[g] + BM - 1) / BM : 0; };
+    int total = 0;
+    for (int g0 = 0; g0 < p.batch; g0 += 64)
+    {
+        int t = tiles_of(g0 + lane);
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1)
+            t += __shfl_xor(t, d, 64);
+        total += t;
+    }
+    total = __builtin_amdgcn_readfirstlane(total) * tiles_n;
+    if (wg >= total)
+        return {-1, 0};
+    const int q = total >> 3, r = total & 7, xcd = wg & 7;
+    const int id = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (wg >> 3);
+    int before = 0;
+    for (int g0 = 0; g0 < p.batch; g0 += 64)
+    {
+        const int t = tiles_of(g0 + lane);
+        int incl = t;
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1)
+        {
+            const int o = __shfl_up(incl, d, 64);
+            incl += lane >= d ? o : 0;
+        }
+        const bool mine = id < (before + incl) * tiles_n; // from the group that holds it on
+        const uint64_t mask = __builtin_amdgcn_ballot_w64(mine);
+        if (mask != 0)
+        {
+            const int at = __builtin_ctzll(mask);
+            return {__builtin_amdgcn_readfirstlane(g0 + at), __builtin_amdgcn_readfirstlane(id - (before + __shfl(incl - t, at, 64)) * tiles_n)};
+        }
+        before += __shfl(incl, 63, 64);
+    }
+    return {-1, 0};
+}
+
 // LW > 0: LW extra waves that do nothing but issue the LDS-DMA.  One wave sustains about one LDS-DMA instruction per ~150
 // cycles whatever else it does (the instruction holds its issuer for 100 - 185 cycles), which in the 8-wave 256 x 192 shape is a
 // third of every compute wave's issue time; loaders (the shape's 160 VGPRs leave room for a third wave per SIMD) take that
@@ -69,18 +120,27 @@ template <int WT, int WM, int WN, int MT, int NT, int KG, int BKB, int S, int LW
 __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(const GemmParams p_in)
 {
     GemmParams p = p_in;
+    int group_wg = 0; // grouped: the tile inside this workgroup's group
     if constexpr (WT == W_BF16)
     {
         // a batch of independent products of one shape (the stack engine's per-head products): blockIdx.y picks the operands
-        p.a = reinterpret_cast<const char*>(p.a) + (int64_t) blockIdx.y * p.batch_a;
-        p.w = reinterpret_cast<const char*>(p.w) + (int64_t) blockIdx.y * p.batch_w;
-        p.c = reinterpret_cast<char*>(p.c) + (int64_t) blockIdx.y * p.batch_c;
+        // (a grouped product has one grid over the tiles its groups really have: see below)
+        int64_t prod = blockIdx.y;
         if (p.group_off)
         {
-            const int64_t o = p.group_off[blockIdx.y];
-            p.M = p.group_off[blockIdx.y + 1] - (int) o;
-            if (p.M <= 0)
-                return;
+            const GroupTile gt = group_tile<WM * MT * 32>(p, (p.N + WN * NT * 32 - 1) / (WN * NT * 32), (int) blockIdx.x);
+            if (gt.group < 0)
+                return; // behind the last tile
+            prod = gt.group;
+            group_wg = gt.tile;
+        }
+        p.a = reinterpret_cast<const char*>(p.a) + prod * p.batch_a;
+        p.w = reinterpret_cast<const char*>(p.w) + prod * p.batch_w;
+        p.c = reinterpret_cast<char*>(p.c) + prod * p.batch_c;
+        if (p.group_off)
+        {
+            const int64_t o = p.group_off[prod];
+            p.M = p.group_off[prod + 1] - (int) o;
             if (p.a_rows)
                 p.a_rows += o;
             else
@@ -119,9 +179,9 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
     // contiguous range of tiles so that the tiles sharing an A row-panel / W column-panel share an L2
     const int nwg = gridDim.x;
     int wg = blockIdx.x;
-    // (a grouped product has fewer tiles than the grid, the first ids: in launch order they already go round the XCDs, while
-    // contiguous ranges per XCD would leave every group's tiles on the first XCDs)
-    if (!(WT == W_BF16 && p.group_off))
+    if (WT == W_BF16 && p.group_off)
+        wg = group_wg;
+    else
     {
         const int q = nwg >> 3, r = nwg & 7, xcd = wg & 7, idx = wg >> 3;
         wg = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + idx;
@@ -130,11 +190,6 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
     const int tm = wg % tiles_m, tn = wg / tiles_m; // M fastest: the (few) row panels of one W panel run together
     const int m0 = tm * BM, n0 = tn * BN;
     const int M = p.M, N = p.N;
-    if constexpr (WT == W_BF16)
-    {
-        if (n0 >= N)
-            return; // a group with fewer rows than the launch's bound has fewer tiles than the grid
-    }
     const int ntile = (p.K * ES) / BKB;
 
     // ---- DMA source addresses: chunk c (RPC tile rows) -> lane l: row c * RPC + l / PPR, LDS piece l % PPR
@@ -555,7 +610,14 @@ int launch_cfg(const GemmParams& p, hipStream_t stream)
     auto kfn = gemm_glds_kernel<WT, WM, WN, MT, NT, KG, BKB, S, LW>;
     launch_util::ensure_dynamic_lds(reinterpret_cast<const void*>(kfn), smem);
     const int tiles = ((p.M + BM - 1) / BM) * ((p.N + BN - 1) / BN);
-    hipLaunchKernelGGL(kfn, dim3(tiles, WT == W_BF16 && p.batch > 1 ? p.batch : 1), dim3(64 * (WM * WN * KG + LW)), smem, stream, p);
+    dim3 grid(tiles, WT == W_BF16 && p.batch > 1 ? p.batch : 1);
+    if (WT == W_BF16 && p.group_off)
+    {
+        // at most this many row tiles: full ones, and one begun in every group that has rows
+        const int64_t rows = p.group_total;
+        grid = dim3((unsigned) ((rows / BM + std::min<int64_t>(p.batch, rows)) * ((p.N + BN - 1) / BN)));
+    }
+    hipLaunchKernelGGL(kfn, grid, dim3(64 * (WM * WN * KG + LW)), smem, stream, p);
     hipError_t e = hipGetLastError();
     if (e != hipSuccess)
     {

@@ -395,6 +395,7 @@ struct GemmParams
     // ... grouped: device int32 [batch + 1]; product b takes rows [group_off[b], group_off[b + 1]) of a and c (batch_a = batch_c = 0), M
     // is the host's bound on a group's rows
     const int32_t* group_off = nullptr;
+    int32_t group_total = 0;         // grouped: the most rows all groups together have (sizes the grid)
     const int32_t* a_rows = nullptr; // grouped: row r of the products' common row range reads a's row a_rows[r]
     // microbench hook (tllm_gemm_set_clock_probe), set by the launchers only: 2 x uint64 per workgroup {shader cycles, 100 MHz ticks}
     void* clock_probe = nullptr;

@@ -463,15 +463,45 @@ __global__ __launch_bounds__(1024) void argmax_kernel(int32_t* out_ids, const fl
     const float* l = logits + (int64_t) blockIdx.x * vocab;
     float best = -INFINITY;
     int bi = 0x7fffffff;
-    for (int i = threadIdx.x; i < vocab; i += blockDim.x)
+    if ((vocab & 3) == 0 && !(reinterpret_cast<uintptr_t>(l) & 15))
     {
-        const float v = l[i];
-        if (v > best || (v == best && i < bi))
+        // 16-byte pieces, four requested before the first is looked at (a piece beyond the row: the last one again); a thread's indices
+        // only grow, so an equal later value never replaces an earlier one
+        const int n4 = vocab >> 2;
+        for (int i0 = threadIdx.x; i0 < n4; i0 += 4 * (int) blockDim.x)
         {
-            best = v;
-            bi = i;
+            float4 v[4];
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+            {
+                const int i = i0 + k * (int) blockDim.x;
+                v[k] = reinterpret_cast<const float4*>(l)[i < n4 ? i : n4 - 1];
+            }
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+            {
+                const int i = i0 + k * (int) blockDim.x;
+                const float e[4] = {v[k].x, v[k].y, v[k].z, v[k].w};
+#pragma unroll
+                for (int c = 0; c < 4; ++c)
+                    if (i < n4 && (e[c] > best || (e[c] == best && 4 * i + c < bi)))
+                    {
+                        best = e[c];
+                        bi = 4 * i + c;
+                    }
+            }
         }
     }
+    else
+        for (int i = threadIdx.x; i < vocab; i += blockDim.x)
+        {
+            const float v = l[i];
+            if (v > best || (v == best && i < bi))
+            {
+                best = v;
+                bi = i;
+            }
+        }
 #pragma unroll
     for (int m = 32; m >= 1; m >>= 1)
     {

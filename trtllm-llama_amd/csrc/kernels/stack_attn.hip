@@ -873,16 +873,26 @@ __global__ __launch_bounds__(64) void attn_split_merge_kernel(const StackAttnPar
 #pragma unroll
         for (int m = 0; m < MAPS; ++m)
             a[c][m] = 0.f;
-#pragma unroll
-    for (int i = 0; i < kMaxSplits * MAPS; ++i)
+    // four partials at a time, every load of them requested before the first is used (partials beyond the last: the last again, weight 0)
+    const int n_part = ks * MAPS;
+    for (int i0 = 0; i0 < n_part; i0 += 4)
     {
-        const float wgt = __shfl(wl, i, 64);
-        if (i < ks * MAPS) // wave-uniform
+        float v[4][MC];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
         {
+            const float* part = base + (int64_t) (i0 + j < n_part ? i0 + j : n_part - 1) * (V + 2);
 #pragma unroll
             for (int c = 0; c < MC; ++c)
-                if (lane + c * 64 < V)
-                    a[c][i % MAPS] += wgt * base[i * (V + 2) + lane + c * 64];
+                v[j][c] = part[lane + c * 64 < V ? lane + c * 64 : V - 1];
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+        {
+            const float wgt = i0 + j < n_part ? __shfl(wl, i0 + j, 64) : 0.f;
+#pragma unroll
+            for (int c = 0; c < MC; ++c)
+                a[c][j % MAPS] += wgt * v[j][c]; // (i0 is a multiple of 4: partial i0 + j belongs to map j % MAPS)
         }
     }
 #pragma unroll

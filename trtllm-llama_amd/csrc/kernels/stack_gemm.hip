@@ -108,7 +108,7 @@ __global__ __launch_bounds__(256) void fma_tile_kernel(const StackGemmParams p_i
         {
             const int idx = tid + i * 256, r = idx / TK, k = idx % TK;
             As[k][r] = (m0 + r < p.M && k0 + k < p.K) ? ld_el<DT>(p.a, row_s[r] + k0 + k) : 0.f;
-            Ws[k][r] = (n0 + r < p.N && k0 + k < p.K) ? ld_el<DT>(p.w, (int64_t) (n0 + r) * p.K + k0 + k) : 0.f;
+            Ws[k][r] = (n0 + r < p.N && k0 + k < p.K) ? ld_el<DT>(p.w, (int64_t) (n0 + r) * p.ldw + k0 + k) : 0.f;
         }
         __syncthreads();
 #pragma unroll
@@ -168,7 +168,7 @@ __global__ __launch_bounds__(256) void skinny_kernel(const StackGemmParams p_in)
         uint4 wv[SK_R];
 #pragma unroll
         for (int r = 0; r < SK_R; ++r)
-            wv[r] = n0 + r < p.N ? ld_nt16(w + (int64_t) (n0 + r) * p.K + k) : make_uint4(0, 0, 0, 0);
+            wv[r] = n0 + r < p.N ? ld_nt16(w + (int64_t) (n0 + r) * p.ldw + k) : make_uint4(0, 0, 0, 0);
 #pragma unroll
         for (int m = 0; m < MR; ++m)
         {
@@ -198,6 +198,18 @@ __global__ __launch_bounds__(256) void skinny_kernel(const StackGemmParams p_in)
             if (lane == 0 && m < p.M && n0 + r < p.N)
                 seam<DT_BF16>(p, m, n0 + r, s);
         }
+}
+
+// the parts of a product cut along K: their sum, in the order of K, through the product's epilogue
+__global__ __launch_bounds__(256) void split_sum_kernel(const StackGemmParams p, const float* ws, int parts)
+{
+    const int64_t i = (int64_t) blockIdx.x * 256 + threadIdx.x, n = (int64_t) p.M * p.N;
+    if (i >= n)
+        return;
+    float v = 0.f;
+    for (int k = 0; k < parts; ++k)
+        v += ws[(int64_t) k * n + i];
+    seam<DT_BF16>(p, (int) (i / p.N), (int) (i % p.N), v);
 }
 
 inline int launched(const char* what)
@@ -263,10 +275,13 @@ int launch_glds_bf16(const GemmParams& g, hipStream_t stream, int m_expected = 0
 
 } // namespace
 
-int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
+int launch_stack_gemm(const StackGemmParams& p_in, hipStream_t stream)
 {
+    StackGemmParams p = p_in;
     if (p.M <= 0 || p.N <= 0)
         return 0;
+    if (p.ldw == 0)
+        p.ldw = p.K;
     if (p.K <= 0 || !p.a || !p.w || (!p.c && !p.resid))
     {
         set_error("stack_gemm: M %d N %d K %d with a missing operand", p.M, p.N, p.K);
@@ -278,7 +293,7 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
         return -1;
     }
     if (p.batch < 1 || (p.batch > 1 && p.resid) || (p.group_off && (p.resid || p.stride_a || p.stride_c))
-        || (p.a_rows && !p.group_off) || p.seam.n_sec < 0 || p.seam.n_sec > 2 || (p.seam.n_sec > 0 && (p.batch > 1 || p.group_off || p.resid))
+        || (p.a_rows && !p.group_off) || (p.group_off && p.group_total < 1) || p.ldw < p.K || p.seam.n_sec < 0 || p.seam.n_sec > 2 || (p.seam.n_sec > 0 && (p.batch > 1 || p.group_off || p.resid))
         || (p.act == ACT_GELU_MUL && (!p.seam.mul || !p.seam.mul_rows || p.group_off)))
     {
         set_error("stack_gemm: batch %d, act %d (a batched product has no residual seam and no output sections; a grouped one takes its rows from one a and one c)", p.batch, p.act);
@@ -290,7 +305,7 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
         hipLaunchKernelGGL((fma_tile_kernel<DT_FLOAT>), tiles, dim3(256), 0, stream, p);
         return launched("stack_gemm fp32");
     }
-    const bool aligned = !(reinterpret_cast<uintptr_t>(p.a) & 15) && !(reinterpret_cast<uintptr_t>(p.w) & 15) && p.K % 8 == 0 && p.lda % 8 == 0
+    const bool aligned = !(reinterpret_cast<uintptr_t>(p.a) & 15) && !(reinterpret_cast<uintptr_t>(p.w) & 15) && p.K % 8 == 0 && p.lda % 8 == 0 && p.ldw % 8 == 0
         && (p.batch == 1 || (p.stride_a % 8 == 0 && p.stride_w % 8 == 0));
     if (aligned && p.M <= 8)
     {
@@ -302,6 +317,37 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
         else
             hipLaunchKernelGGL((skinny_kernel<8>), grid, dim3(256), 0, stream, p);
         return launched("stack_gemm skinny");
+    }
+    const int64_t tiles128 = (int64_t) ((p.M + 127) / 128) * ((p.N + 127) / 128);
+    if (aligned && p.split_ws && p.batch == 1 && p.M >= 32 && tiles128 * 2 <= launch_util::device_cus())
+    {
+        // few tiles: parts of K (whole 128-byte stages, at least 4 of them) until the chip is full
+        int parts = 1;
+        while (parts < 16 && tiles128 * parts * 2 <= launch_util::device_cus() && p.K % (64 * parts * 2) == 0 && p.K / (parts * 2) >= 256
+            && (int64_t) parts * 2 * p.M * p.N <= p.split_floats)
+            parts *= 2;
+        if (parts > 1)
+        {
+            StackGemmParams part;
+            part.dtype = p.dtype;
+            part.out_f32 = 1;
+            part.M = p.M;
+            part.N = p.N;
+            part.K = p.K / parts;
+            part.a = p.a;
+            part.lda = p.lda;
+            part.w = p.w;
+            part.ldw = p.ldw;
+            part.c = p.split_ws;
+            part.ldc = p.N;
+            part.batch = parts;
+            part.stride_a = part.stride_w = part.K;
+            part.stride_c = (int64_t) p.M * p.N;
+            if (launch_stack_gemm(part, stream))
+                return -1;
+            hipLaunchKernelGGL(split_sum_kernel, dim3((unsigned) (((int64_t) p.M * p.N + 255) / 256)), dim3(256), 0, stream, p, p.split_ws, parts);
+            return launched("stack_gemm split sum");
+        }
     }
     if (aligned && (!p.group_off || p.K % 64 == 0))
     {
@@ -321,7 +367,7 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
             g.a = reinterpret_cast<const char*>(p.a) + (int64_t) b * p.stride_a * 2;
             g.lda = p.lda;
             g.w = reinterpret_cast<const char*>(p.w) + (int64_t) b * p.stride_w * 2;
-            g.ldw = (int64_t) p.K * 2;
+            g.ldw = p.ldw * 2;
             g.c = p.c ? reinterpret_cast<char*>(p.c) + (int64_t) b * p.stride_c * (p.out_f32 ? 4 : 2) : nullptr;
             g.ldc = p.ldc;
             g.resid = p.resid;
@@ -340,6 +386,7 @@ int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream)
                 g.batch_w = p.stride_w * 2;
                 g.batch_c = p.stride_c * (p.out_f32 ? 4 : 2);
                 g.group_off = p.group_off;
+                g.group_total = p.group_total;
                 rc = launch_glds_bf16(g, stream, p.group_off ? p.group_rows : 0);
             }
             else

@@ -42,6 +42,11 @@ struct StackGemmParams
     const void* a = nullptr;
     int64_t lda = 0;             // elements
     const void* w = nullptr;     // [N, K] row-major, K contiguous
+    int64_t ldw = 0;             // elements between rows of w, 0: K
+    // optional room for fp32 partial products (split_floats of them): a product with too few tiles to fill the chip is cut along K, the
+    // parts run as one batch and a second launch sums them and applies the epilogue
+    float* split_ws = nullptr;
+    int64_t split_floats = 0;
     void* c = nullptr;
     int64_t ldc = 0;
     float* resid = nullptr;      // fp32 [M, ldr]
@@ -58,6 +63,7 @@ struct StackGemmParams
     const int32_t* group_off = nullptr;
     const int32_t* a_rows = nullptr; // grouped: row r of the common row range reads a's row a_rows[r] (device; no copy of the rows in group order)
     GemmSeam seam;
+    int32_t group_total = 0; // the most rows all groups together have
     int32_t group_rows = 0; // the rows a group is expected to have (tile shapes are chosen for it), 0: M
 };
 int launch_stack_gemm(const StackGemmParams& p, hipStream_t stream);

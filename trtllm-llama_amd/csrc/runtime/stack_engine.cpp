@@ -73,6 +73,8 @@ enum MlpKind
     MLP_MOE = 2        // routed experts of size ff - W_down (silu(W_gate h) * W_up h) or W_down relu(W_up h)^2 -, the last `identity` router
                        // outputs return h; optionally a shared expert of size shared_ff that every token uses
 };
+constexpr int kSideParts = 16; // the token input's gate product has few columns: room for this many parts of its K
+
 struct HyperW
 {
     float *mix = nullptr, *out = nullptr, *in = nullptr;
@@ -142,7 +144,7 @@ struct tllm_stack
     int embed_norm = 0, loop_input = 1, side_dim = 0;
     float logit_scale = 1.f, logit_cap = 0.f;
     void *side_embed = nullptr, *x_el = nullptr, *side_act = nullptr, *act_sh = nullptr;
-    float *embed_norm_w = nullptr, *route_z = nullptr;
+    float *embed_norm_w = nullptr, *route_z = nullptr, *split_ws = nullptr;
     int streams = 1;
     float norm_offset = 0.f, *ones = nullptr;
     float eps = 1e-5f, emb_scale = 1.f;
@@ -181,13 +183,13 @@ struct tllm_stack
     }
     void free_scratch()
     {
-        void* all[] = {x_el, side_act, act_sh, route_z, x, x0, o32, logits, tap, y32, h1, h2, proj, q, ctx, act, hw, lat, ints, ids_out, xbc, cq, qfull, moe_a, moe_y, moe_w, moe_i,
+        void* all[] = {split_ws, x_el, side_act, act_sh, route_z, x, x0, o32, logits, tap, y32, h1, h2, proj, q, ctx, act, hw, lat, ints, ids_out, xbc, cq, qfull, moe_a, moe_y, moe_w, moe_i,
             h32, dl_a, dl_g, pairs};
         for (void* p : all)
             if (p)
                 (void) hipFree(p);
         x_el = side_act = act_sh = nullptr;
-        route_z = nullptr;
+        route_z = split_ws = nullptr;
         x = x0 = o32 = logits = tap = y32 = nullptr;
         h1 = h2 = proj = q = ctx = act = hw = lat = nullptr;
         ints = ids_out = nullptr;
@@ -339,6 +341,7 @@ int ensure_scratch(tllm_stack* s, int tokens, int want, int n_ints)
         HIP_OK(hipMalloc(&s->x_el, (s->side_dim ? T * wd : 1) * es));
         HIP_OK(hipMalloc(&s->act_sh, T * std::max(s->max_sh, 1) * es));
         HIP_OK(hipMalloc((void**) &s->route_z, (s->plain ? T * std::max(s->max_outputs, 1) : 1) * 4));
+        HIP_OK(hipMalloc((void**) &s->split_ws, T * (size_t) std::max(s->side_dim, 1) * kSideParts * 4));
         HIP_OK(hipMalloc(&s->side_act, T * std::max(s->side_dim, 1) * es));
         HIP_OK(hipMalloc(&s->hw, W * wd * es));
         HIP_OK(hipMalloc((void**) &s->ints, NI * 4));
@@ -1659,6 +1662,7 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         u.batch = l.experts;
         u.stride_w = (int64_t) up_cols * Wd;
         u.group_off = mp.group_off;
+        u.group_total = (int) pairs;
         u.group_rows = (int) std::min<int64_t>(T, (pairs + l.experts - 1) / l.experts);
         if (launch_stack_gemm(u, stream)
             || (!l.expert_relu2 && launch_stack_gelu_gate(s->act, s->proj, s->dtype, (int) pairs, l.ff, u.N, stream, GATE_SILU)))
@@ -1677,6 +1681,7 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
         dn.batch = l.experts;
         dn.stride_w = (int64_t) Wd * l.ff;
         dn.group_off = mp.group_off;
+        dn.group_total = u.group_total;
         dn.group_rows = u.group_rows;
         return (launch_stack_gemm(dn, stream) || launch_stack_moe_combine(mp, s->moe_y, y, stream)) ? -1 : 0;
     };
@@ -1788,6 +1793,8 @@ int32_t tllm_stack_step(tllm_stack_t s, const tllm_stack_batch_t* b, float* logi
                 sg.w = l.side_gate;
                 sg.c = s->side_act;
                 sg.ldc = s->side_dim;
+                sg.split_ws = s->split_ws;
+                sg.split_floats = (int64_t) s->cap_tokens * s->side_dim * kSideParts;
                 sg.act = ACT_GELU_MUL;
                 sg.seam.mul = (const char*) s->side_embed + (size_t) r.layer * s->side_dim * s->es;
                 sg.seam.mul_rows = d_tok;
