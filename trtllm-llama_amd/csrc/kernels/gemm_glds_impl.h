@@ -536,6 +536,48 @@ __global__ __launch_bounds__(64 * (WM * WN * KG + LW)) void gemm_glds_kernel(con
         }
         return;
     }
+    if constexpr (WT == W_BF16 && LW == 0 && KG == 1)
+    {
+        // plain fp32 rows (stored, or added to the residual stream): a 32 x 32 block at a time through the wave's LDS scratch, 16 bytes per
+        // lane and access.  Element by element this was the longest part of a short product.
+        const bool plain = !p.bias && !p.act && !(N & 3) && !(p.seam.n_sec > 0 && n0 + BN > p.seam.sec[0].col0);
+        float* dst = p.resid ? (p.gate ? nullptr : p.resid) : (p.out_dtype == DT_FLOAT ? reinterpret_cast<float*>(p.c) : nullptr);
+        const int64_t ldd = p.resid ? p.ldr : p.ldc;
+        if (plain && dst && !(ldd & 3) && !(reinterpret_cast<uintptr_t>(dst) & 15))
+        {
+            constexpr int P4 = 36; // floats per scratch row: 16-byte aligned, rows spread over the banks
+            static_assert(32 * P4 * 4 <= 32 * (NT * 64 + 16), "the scratch of a wave");
+            __syncthreads(); // every wave has finished reading the operand buffers
+            float* scr = reinterpret_cast<float*>(lds + wid * (32 * (NT * 64 + 16)));
+#pragma unroll
+            for (int i = 0; i < MT; ++i)
+#pragma unroll
+                for (int j = 0; j < NT; ++j)
+                {
+#pragma unroll
+                    for (int r = 0; r < 16; ++r)
+                        scr[((r & 3) + 8 * (r >> 2) + 4 * (lane >> 5)) * P4 + (lane & 31)] = acc[i][j][r];
+#pragma unroll
+                    for (int s = 0; s < 4; ++s)
+                    {
+                        const int rr = (lane >> 3) + s * 8, pc = (lane & 7) * 4;
+                        float4 v = *reinterpret_cast<const float4*>(scr + rr * P4 + pc);
+                        const int grow = m0 + (wm * MT + i) * 32 + rr, gcol = wave_n0 + j * 32 + pc;
+                        if (grow < M && gcol < N)
+                        {
+                            float4* at = reinterpret_cast<float4*>(dst + (int64_t) grow * ldd + gcol);
+                            if (p.resid)
+                            {
+                                const float4 o = *at;
+                                v = make_float4(o.x + v.x, o.y + v.y, o.z + v.z, o.w + v.w);
+                            }
+                            *at = v;
+                        }
+                    }
+                }
+            return;
+        }
+    }
 #pragma unroll
     for (int i = 0; i < MT; ++i)
 #pragma unroll
