@@ -483,8 +483,10 @@ __global__ __launch_bounds__(NW * 64) void attn_tile_kernel(const StackAttnParam
 // number of 16-byte pieces, V^T rows to 80 bytes: the fragment reads spread over the banks) - the next block's global loads are in
 // flight while this block is computed.  Same transposed products and operand slots as attn_tile_kernel; no merge: a wave finishes
 // its own rows (lambda combination, head norm, bfloat16 store).  Tiles are handed out heaviest first (the last rows see most keys).
+// Two waves per SIMD where the registers allow it: with the whole file to one wave the compiler keeps the accumulators in the
+// accumulation registers and moves all of them back and forth around every block's softmax.
 template <int MAPS, int DK, int VT>
-__global__ __launch_bounds__(256) void attn_prefill_kernel(const StackAttnParams p, int min_count)
+__global__ __launch_bounds__(256, DK >= 10 ? 1 : 2) void attn_prefill_kernel(const StackAttnParams p, int min_count)
 {
     constexpr int D = DK * 32, V = VT * 16;
     constexpr int KP = D * 2 + 16, VP = 80;                 // LDS row pitches in bytes
@@ -794,9 +796,8 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
                 {
                     const bf16x8 kfr = as_bf16x8(*reinterpret_cast<const uint4*>(k_s + (t * 16 + col) * KP + (ks * 32 + 8 * g4) * 2));
 #pragma unroll
-                    for (int rt = 0; rt < RT; ++rt)
-                        if (on[rt])
-                            s[rt][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kfr, qf[rt][ks], s[rt][t], 0, 0, 0);
+                    for (int rt = 0; rt < RT; ++rt) // (no branches among the products: a tile that is off has its scores dropped below)
+                        s[rt][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kfr, qf[rt][ks], s[rt][t], 0, 0, 0);
                 }
             uint4 pf[RT];
 #pragma unroll
@@ -818,8 +819,7 @@ __global__ __launch_bounds__(256) void attn_prefill_wide_kernel(const StackAttnP
                 const bf16x8 vf = as_bf16x8(make_uint4(lo.x, lo.y, hi.x, hi.y));
 #pragma unroll
                 for (int rt = 0; rt < RT; ++rt)
-                    if (on[rt])
-                        acc[rt][ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, as_bf16x8(pf[rt]), acc[rt][ct], 0, 0, 0);
+                    acc[rt][ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, as_bf16x8(pf[rt]), acc[rt][ct], 0, 0, 0);
             }
         }
         __syncthreads();
@@ -937,8 +937,9 @@ int launch_tile(const StackAttnParams& p, hipStream_t stream)
         if constexpr (MAPS == 1 && DK >= 5)
         {
             const char* force = std::getenv("TLLM_STACK_WIDE_PREFILL"); // test / measurement knob: 1 = always, 0 = never
+            // (shapes whose 64-row form fits two waves per SIMD run that one: twice the waves hide what the wide form saves in LDS reads)
             wide = !p.head_norm
-                && (force ? force[0] == '1' : (int64_t) ((p.max_count + 127) / 128) * p.entries * p.heads >= launch_util::device_cus());
+                && (force ? force[0] == '1' : DK >= 10 && (int64_t) ((p.max_count + 127) / 128) * p.entries * p.heads >= launch_util::device_cus());
         }
         if constexpr (MAPS == 1 && DK >= 5)
         {
