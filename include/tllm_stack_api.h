@@ -17,15 +17,20 @@
  * learned matrix after the softmax, a gate per output channel, weighted q / k norms, three-band frequency scaling, an output bias),
  * "latent_attention" (keys and values expanded from one low-rank latent per token plus one rotated key part shared by the
  * heads; the cache holds the latent and that part, attention runs in the absorbed form; optionally queries expanded from a normed
- * latent of their own, half-split rotation pairs with YaRN-style frequency scaling, a window or chunk mask, a softmax sink), "hgrn2"
+ * latent of their own, half-split rotation pairs with YaRN-style frequency scaling, a window or chunk mask, a softmax sink, a per-head output
+ * gate), "hgrn2"
  * (gated linear recurrence with a lower-bounded forget gate, fp32 state) and "mamba2" (selective state-space layer: a short causal
  * convolution whose last inputs are part of the state, S <- exp(-exp(A_log) dt) S + dt B x^T per head over grouped B / C, skip, gate,
  * RMS norm in parts of the row) and "delta_rule" (gated delta rule with a decay per key channel: q | k | v through a short causal
  * convolution and silu, unit q and k, S <- diag(g) S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; RMS norm per head and a low-rank
  * sigmoid gate).  The embedding may add a hashed row per (previous token, token) pair, and every mixer's normed input may be blended
- * with the previous token's (token shift); both carry one item per sequence in its state slot.  Feed-forwards: gated dense, relu^2, or a routed mixture of gated experts (softmax router with a
- * choice correction, groups of experts of which only the best can be chosen, identity experts).  A layer may run on an earlier
- * layer's weights (layer.<i>.weights_of), with a cache / state of its own.  Two block forms: parallel sublayers on one residual whose updates are gated by
+ * with the previous token's (token shift); both carry one item per sequence in its state slot.  Feed-forwards: gated dense, relu^2, or a routed mixture of gated or relu^2 experts (softmax or sigmoid
+ * router with a choice correction, groups of experts of which only the best can be chosen, identity experts, weights divided by their
+ * sum, a shared expert for every token).  A layer may run on an earlier
+ * layer's weights (layer.<i>.weights_of), with a cache / state of its own.  Three block forms: parallel sublayers on one plain residual that both read one normed
+ * row (the stream may start from a normed embedding row, and every layer may end with a token input: the layer's part of a per-token
+ * side embedding, gated by a projection of the stream, projected back and RMS-normed; loops as below, without the range's input);
+ * parallel sublayers on one residual whose updates are gated by
  * sigmoid(W h + b), RMS norms in groups, a range of layers optionally run several times in a row (every pass with a cache / state
  * of its own); or sequential pre-norm sublayers on `streams` hyper-connected residual copies (u = sum_s in[s] x_s feeds the
  * sublayer, x_t <- sum_s mix[s, t] x_s + out[t] y lands its result; the output norm reads sum_s x_s).
@@ -50,7 +55,10 @@ typedef struct tllm_stack* tllm_stack_t;
 /* Configuration text, one key=value per line:
  *   dtype (bfloat16 | float32), width, vocab, num_layers, norm_groups (1), norm_eps (1e-5), embedding_scale (1),
  *   loop_start, loop_stop, loop_times (0, 0, 1: no loop), page_size (64), num_blocks, num_slots, debug_taps (0),
- *   block (parallel | sequential), residual (gated | hyper; parallel goes with gated, sequential with hyper), streams (1 .. 8),
+ *   block (parallel | sequential), residual (gated | hyper | plain; parallel goes with gated or plain, sequential with hyper), streams (1 .. 8),
+ *   loop_input (1 | 0: later passes over a looped range do not add what the first pass started from; 0 with residual=plain),
+ *   embedding_norm (0 | 1: tensor embed.norm; residual=plain), token_side (0: none; channels of a layer's token input; residual=plain),
+ *   logit_scale (1), logit_softcap (0: none; logits <- cap tanh(scale z / cap)),
  *   norm_offset (0: a norm weight is applied as norm_offset + stored value),
  *   pair_buckets (0: none; the tensor `bigram` [pair_buckets + 1, width] adds row (prev * pair_mul_prev + token * pair_mul_cur) mod
  *     pair_buckets to a token's embedding, its last row to a sequence's first token), pair_mul_prev, pair_mul_cur,
@@ -61,7 +69,8 @@ typedef struct tllm_stack* tllm_stack_t;
  *       W_down (silu(W_gate h) * W_up h) of size .ff plus .identity identity outputs, .top chosen per token among the .route_keep best
  *       of .route_groups equal groups, weights = softmax score * .route_scale; .route_score softmax | sigmoid (every output's
  *       score by itself), .route_weight output | input (an expert runs on weight x row and the outputs are summed as they
- *       are); relu2 and moe in sequential blocks only),
+ *       are); gated blocks have gelu_gate only, plain ones moe only; .expert silu_gate | relu2 (W_down relu(W_up h)^2), .route_norm
+ *       (0 | 1: weights over their sum + 1e-20), .shared_ff (0: none; size of the shared expert, relu2 form)),
  *     attention: .kv_heads, .maps (1 | 2), .diff (the constant of the second map's weight and of the output scale 1 - diff),
  *       .scale, .softcap (0: none), .head_norm (0 | 1), .rot_dims, .rot_base, .rot_factor (0: no frequency scaling),
  *       .rot_original, .rot_fast, .rot_slow, .qkv_bias (0 | 1), .qk_norm (0 | 1: q and k / their RMS over dim), .head_temp (0 | 1),
@@ -72,15 +81,15 @@ typedef struct tllm_stack* tllm_stack_t;
  *       .qk_norm_weight (0 | 1: mix.q.norm / mix.k.norm [dim]), .o_bias (0 | 1), .rot_scaling (yarn | banded: .rot_low, .rot_high);
  *     latent_attention: .kv_rank, .rot_dim (size of the shared rotated part), .rot_dims (how many of them turn), .rot_base, .scale,
  *       .q_rank (0: queries straight from the input), .rot_pairing (neighbours | halves), .rot_factor / .rot_original / .rot_fast /
- *       .rot_slow, .mask, .mask_size, .sink;
+ *       .rot_slow, .mask, .mask_size, .sink, .out_gate (0 | 1);
  *     mamba2: .state (rows of a head's state; takes the place of .dim), .groups, .conv (taps), .ssm_norm_groups;
  *     delta_rule: .kv_heads (q / k heads), .conv (taps), .decay_rank, .gate_rank (of the two low-rank pairs).
  * Weights are named l<i>.norm1, l<i>.norm2, l<i>.mix.{q,k,v,o,lq1,lk1,lq2,lk2} (attention; with the options also q.b, k.b, v.b,
  * temp, r1, r2, sink, pb, g, talk, q.norm, k.norm, o.b), l<i>.mix.{q,dkv,dkv.norm,uk,uv,o} (latent_attention; with a query latent dq, dq.norm, uq instead of q;
- * sink), l<i>.mix.{q,f,f.b,lower,v,norm,o} (hgrn2), l<i>.mix.{in,conv,conv.b,dt_bias,A_log,D,norm,o} (mamba2),
+ * sink, g), l<i>.mix.{q,f,f.b,lower,v,norm,o} (hgrn2), l<i>.mix.{in,conv,conv.b,dt_bias,A_log,D,norm,o} (mamba2),
  * l<i>.mix.{q,k,v,q.conv,k.conv,v.conv,b,a1,a2,dt_bias,A_log,g1,g2,norm,o} (delta_rule), l<i>.shift (token shift), bigram,
- * l<i>.mlp.{gate,up,down} (moe: l<i>.mlp.e<k>.{gate,up,down}, l<i>.mlp.router, l<i>.mlp.correction), l<i>.rg1, l<i>.rg1.b, l<i>.rg2, l<i>.rg2.b (gated residual), l<i>.hc{1,2}.{in,out,mix} (hyper
- * residual; absent with one stream: the plain sum), embed, loop.step, final.norm, head; linear weights [out, in]. */
+ * l<i>.mlp.{gate,up,down} (moe: l<i>.mlp.e<k>.{gate,up,down}, l<i>.mlp.router, l<i>.mlp.correction, l<i>.mlp.shared.{up,down}; relu2 experts have no gate), l<i>.rg1, l<i>.rg1.b, l<i>.rg2, l<i>.rg2.b (gated residual), l<i>.hc{1,2}.{in,out,mix} (hyper
+ * residual; absent with one stream: the plain sum), l<i>.side.{gate,proj,norm}, side.embed [vocab, layers * token_side], embed, embed.norm, loop.step, final.norm, head; linear weights [out, in]. */
 tllm_stack_t tllm_stack_create(const char* config_text);
 
 /* One weight tensor from HOST memory; dtype 0 = fp32, 7 = bfloat16 (nvinfer1::DataType codes).  Converted to the engine's element

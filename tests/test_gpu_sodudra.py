@@ -109,6 +109,7 @@ MECHANISMS = {
     'moe_one_expert': make_config([layer(mlp=moe(experts=1, top=1))]),
     'moe_every_expert': make_config([layer(mlp=moe(experts=4, top=4))]),
     'moe_many_experts': make_config([layer(mlp=moe(experts=70, top=5, ff=9, shared=8))], width=160),
+    'moe_thirty_chosen': make_config([layer(mlp=moe(experts=40, top=30, ff=8, shared=16))], width=128),
     'moe_sixteen_chosen': make_config([layer(mlp=moe(experts=20, top=16, ff=8, shared=16))], width=128),
     'moe_equal_shared_and_expert_size': make_config([layer(mlp=moe(ff=32, shared=32))]),
     'moe_tile_sizes': make_config([layer(heads=2, dim=32, vdim=32, kv_rank=32, mlp=moe(experts=4, top=2, ff=128, shared=192))], width=128),
@@ -462,7 +463,7 @@ def test_descriptions_that_cannot_run_are_refused():
     good = as_model(cfg, w).config.engine_config()
     good.update(dtype='float32', num_blocks=2, num_slots=1)
     for change in ({'block': 'sequential'}, {'loop_input': 1}, {'norm_groups': 3}, {'layer.0.mlp': 'gelu_gate'}, {'token_side': -1},
-                   {'layer.0.expert': 'silu_gate'}, {'layer.0.top': 17, 'layer.0.experts': 20}):
+                   {'layer.0.expert': 'silu_gate'}, {'layer.0.top': 65, 'layer.0.experts': 70}):
         with pytest.raises(RuntimeError):
             StackEngine(dict(good, **change), as_tensors(w))
     with pytest.raises(RuntimeError, match='side.proj'):

@@ -959,6 +959,13 @@ int launch_tile(const StackAttnParams& p, hipStream_t stream)
     {
         // a step of decoded tokens only (every entry within one tile, few rows in all): the keys of an (entry, head) are split over
         // ks workgroups so that a long context is walked by ks * NW waves, two key blocks or so each
+        // single decoded tokens whose heads share one key/value head and carry no per-head score numbers: 16 heads are the tile's rows
+        // (a sink or an output gate is looked up per row)
+        const int head_rows = (p.max_count == 1 && p.kv_heads == 1 && !p.cross_values && MAPS == 1 && p.heads >= 8 && !p.temp && !p.slope && !p.log_r1
+                                  && !p.wbias && !p.head_norm)
+            ? 1
+            : 0;
+        const int gz = head_rows ? (p.heads + 15) / 16 : p.heads;
         int ks = 1;
         if (p.split_ws && p.max_count <= 16 && p.tokens <= kSplitRows)
         {
@@ -966,15 +973,12 @@ int launch_tile(const StackAttnParams& p, hipStream_t stream)
             const int span = p.mask == MASK_CAUSAL ? p.max_context
                                                    : std::min(p.max_context, p.mask_size + 31 + (p.mask_keep > 0 ? p.mask_keep + 31 : 0));
             const int nblk = (span + 31) / 32;
+            // two key blocks per wave, or one where that still leaves CUs without work
             ks = std::min(kMaxSplits, (nblk + 2 * NW - 1) / (2 * NW));
+            if (ks * p.entries * gz * 2 <= launch_util::device_cus())
+                ks = std::min(kMaxSplits, (nblk + NW - 1) / NW);
         }
-        // single decoded tokens whose heads share one key/value head and carry no per-head score numbers: 16 heads are the tile's rows
-        // (a sink or an output gate is looked up per row)
-        const int head_rows = (p.max_count == 1 && p.kv_heads == 1 && !p.cross_values && MAPS == 1 && p.heads >= 8 && !p.temp && !p.slope && !p.log_r1
-                                  && !p.wbias && !p.head_norm)
-            ? 1
-            : 0;
-        const dim3 grid(ks > 1 ? ks : (small_rows + 15) / 16, p.entries, head_rows ? (p.heads + 15) / 16 : p.heads);
+        const dim3 grid(ks > 1 ? ks : (small_rows + 15) / 16, p.entries, gz);
         hipLaunchKernelGGL((attn_tile_kernel<MAPS, DK, VT, NW>), grid, dim3(NW * 64), lds, stream, p, PREFILL_ROWS, ks, head_rows);
         if (ks > 1)
             hipLaunchKernelGGL((attn_split_merge_kernel<MAPS>), dim3(p.tokens, p.heads), dim3(64), 0, stream, p, ks, PREFILL_ROWS);

@@ -200,6 +200,63 @@ __global__ __launch_bounds__(256) void skinny_kernel(const StackGemmParams p_in)
         }
 }
 
+// The same for products of few rows of W (a token input's gate): a workgroup per SK_R rows whose 4 waves split K, so that the weights are
+// requested by four times the waves; their sums meet in LDS.
+template <int MR>
+__global__ __launch_bounds__(256) void skinny_ksplit_kernel(const StackGemmParams p)
+{
+    __shared__ float part[4][SK_R][MR];
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int n0 = blockIdx.x * SK_R;
+    float acc[SK_R][MR];
+#pragma unroll
+    for (int r = 0; r < SK_R; ++r)
+#pragma unroll
+        for (int m = 0; m < MR; ++m)
+            acc[r][m] = 0.f;
+    const uint16_t* a = reinterpret_cast<const uint16_t*>(p.a);
+    const uint16_t* w = reinterpret_cast<const uint16_t*>(p.w);
+    for (int k = (wid * 64 + lane) * 8; k < p.K; k += 256 * 8)
+    {
+        uint4 wv[SK_R];
+#pragma unroll
+        for (int r = 0; r < SK_R; ++r)
+            wv[r] = n0 + r < p.N ? ld_nt16(w + (int64_t) (n0 + r) * p.ldw + k) : make_uint4(0, 0, 0, 0);
+#pragma unroll
+        for (int m = 0; m < MR; ++m)
+        {
+            if (m >= p.M)
+                break;
+            const uint4 xv = *reinterpret_cast<const uint4*>(a + (int64_t) m * p.lda + k);
+            const uint32_t xs[4] = {xv.x, xv.y, xv.z, xv.w};
+#pragma unroll
+            for (int r = 0; r < SK_R; ++r)
+            {
+                const uint32_t ws[4] = {wv[r].x, wv[r].y, wv[r].z, wv[r].w};
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                {
+                    acc[r][m] = fmaf(__builtin_bit_cast(float, xs[i] << 16), __builtin_bit_cast(float, ws[i] << 16), acc[r][m]);
+                    acc[r][m] = fmaf(__builtin_bit_cast(float, xs[i] & 0xffff0000u), __builtin_bit_cast(float, ws[i] & 0xffff0000u), acc[r][m]);
+                }
+            }
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < SK_R; ++r)
+#pragma unroll
+        for (int m = 0; m < MR; ++m)
+        {
+            const float s = wave_sum(acc[r][m]);
+            if (lane == 0)
+                part[wid][r][m] = s;
+        }
+    __syncthreads();
+    const int r = threadIdx.x / MR, m = threadIdx.x % MR;
+    if (r < SK_R && m < p.M && n0 + r < p.N)
+        seam<DT_BF16>(p, m, n0 + r, (part[0][r][m] + part[1][r][m]) + (part[2][r][m] + part[3][r][m]));
+}
+
 // the parts of a product cut along K: their sum, in the order of K, through the product's epilogue
 __global__ __launch_bounds__(256) void split_sum_kernel(const StackGemmParams p, const float* ws, int parts)
 {
@@ -310,6 +367,17 @@ int launch_stack_gemm(const StackGemmParams& p_in, hipStream_t stream)
     if (aligned && p.M <= 8)
     {
         const dim3 grid((p.N + 4 * SK_R - 1) / (4 * SK_R), 1, p.batch);
+        if (p.batch == 1 && !p.group_off && (int) grid.x * 2 <= launch_util::device_cus() && p.K >= 2048)
+        {
+            const dim3 kg((p.N + SK_R - 1) / SK_R);
+            if (p.M <= 1)
+                hipLaunchKernelGGL((skinny_ksplit_kernel<1>), kg, dim3(256), 0, stream, p);
+            else if (p.M <= 4)
+                hipLaunchKernelGGL((skinny_ksplit_kernel<4>), kg, dim3(256), 0, stream, p);
+            else
+                hipLaunchKernelGGL((skinny_ksplit_kernel<8>), kg, dim3(256), 0, stream, p);
+            return launched("stack_gemm skinny (K over waves)");
+        }
         if (p.M <= 1)
             hipLaunchKernelGGL((skinny_kernel<1>), grid, dim3(256), 0, stream, p);
         else if (p.M <= 4)

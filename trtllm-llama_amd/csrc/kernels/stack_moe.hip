@@ -60,7 +60,7 @@ __device__ __forceinline__ void wave_argmax(float& v, int& idx)
 
 constexpr int RT = 8;         // tokens per logits workgroup: a router row is read once for all of them
 constexpr int MAX_OUT = 1024; // router outputs (experts + identities)
-constexpr int MAX_TOP = 16;
+constexpr int MAX_TOP = 64;
 constexpr int FEW_TOKENS = 8; // steps of this many tokens or fewer route in one launch and gather inside the sort
 
 // Router logits, fp32: workgroup (x, y) = 4 router rows (one per wave) x RT tokens; lanes split the width in float4 pieces where

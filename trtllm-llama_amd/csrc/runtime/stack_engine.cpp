@@ -539,9 +539,9 @@ tllm_stack_t tllm_stack_create(const char* config_text)
             l.route_sigmoid = rs == "sigmoid";
             l.route_weight_input = rw == "input";
             const int ne = l.experts + l.identity;
-            if (l.experts < 1 || l.identity < 0 || ne > 1024 || l.top < 1 || l.top > 16 || l.top > ne || l.route_groups < 1 || ne % l.route_groups
+            if (l.experts < 1 || l.identity < 0 || ne > 1024 || l.top < 1 || l.top > 64 || l.top > ne || l.route_groups < 1 || ne % l.route_groups
                 || l.route_keep < 1 || l.route_keep > l.route_groups)
-                return fail("moe: experts >= 1, experts + identity <= 1024 in equal route_groups, 1 <= route_keep <= route_groups, top <= 16");
+                return fail("moe: experts >= 1, experts + identity <= 1024 in equal route_groups, 1 <= route_keep <= route_groups, top <= 64");
             s->max_top = std::max(s->max_top, l.top);
             s->max_experts = std::max(s->max_experts, l.experts);
             s->max_outputs = std::max(s->max_outputs, ne);
